@@ -523,7 +523,9 @@ int tv_patch_embed_strided_fwd(const void* pixels, const void* weight,
  * x / y fp32 or bf16.
  * tv_moe_combine_norm_fwd: u = sum_j weights[row][j] * expert_out[pos[row][j]];
  * pos < 0: an identity expert (its output is the residual row).
- * tv_embed_scaled_fwd: x (fp32) and h (dtype, optional) = table[ids] * scale.
+ * tv_embed_scaled_fwd: x (fp32) and h (dtype, optional) = table[ids] * scale
+ *   (+ pos[start[b] + row - cu[b]], b = seq[row], with a position table of max_pos
+ *   rows; a token behind its end gets none: callers check).
  * --------------------------------------------------------------------- */
 int tv_rmsnorm_ex_fwd(const void* x, const void* weight, const void* gate, const float* residual, float* sum, void* y,
                       void* y2, const int* y2_rows, int64_t y2_stride, int64_t rows, int D, int64_t x_stride,
@@ -534,7 +536,45 @@ int tv_moe_combine_norm_fwd(const void* expert_out, const int* pos, const float*
                             int64_t residual_stride, int64_t sum_stride, int64_t y_stride, float eps, float mult,
                             float weight_offset, int out_dtype, int weight_dtype, int y_dtype, void* stream);
 int tv_embed_scaled_fwd(const int64_t* ids, const void* table, float* x, void* h, int64_t rows, int D, int64_t vocab,
-                        float scale, int dtype, void* stream);
+                        float scale, const void* pos, const int* seq, const int* cu, const int* start, int64_t max_pos,
+                        int dtype, void* stream);
+
+/* ------------------------------------------------------------------------
+ * Parallel layers on a 32-bit residual stream (csrc/stream_ops.hip).
+ * tv_norm_shift_fwd:  x' = x + rmsnorm(y) * y_weight (fp32, x_out; y NULL: x' = x);
+ *   h = rmsnorm(x') * gain[0];  hs = h + (h_before - h) * shift (shift NULL: none).
+ *   h_before is the h of the previous row of the same sequence; of a sequence's first
+ *   row: zeros at position 0, else row (position - 1) & 1 of the state block slot[b]
+ *   ((2, D) fp32 blocks, state_stride floats apart); the last row's h goes to its row.
+ *   Row t belongs to sequence seq[t], rows [cu[b], cu[b+1]), start[b] tokens in front.
+ * tv_residual_add_fwd: x_out = x + u (fp32), h (optional) its rounding to dtype.
+ * tv_gated_mul_fwd: o = f(a) * b[b_ids[row]] (b_ids NULL: b[row]; b has b_rows rows);
+ *   act 0: f = sigmoid, 1: f = gelu (tanh form).
+ * tv_scatter_rows: dst[rows_to[r]] = src[r].
+ * dtype fp32 or bf16; x, x_out, state fp32; x and h / hs rows dense.
+ * --------------------------------------------------------------------- */
+int tv_norm_shift_fwd(const float* x, const void* y, const void* y_weight, float* x_out, const void* gain, const void* shift,
+                      float* state, const int* seq, const int* cu, const int* start, const int* slot, void* h, void* hs,
+                      int64_t rows, int D, int64_t y_stride, int64_t state_stride, float eps, int dtype, void* stream);
+int tv_residual_add_fwd(const float* x, const void* u, float* x_out, void* h, int64_t rows, int D, int64_t u_stride,
+                        int dtype, void* stream);
+int tv_gated_mul_fwd(const void* a, const void* b, const int64_t* b_ids, void* o, int64_t rows, int cols, int64_t a_stride,
+                     int64_t b_stride, int64_t o_stride, int64_t b_rows, int act, int dtype, void* stream);
+int tv_scatter_rows(const void* src, const int* rows_to, void* dst, int64_t rows, int cols, int64_t src_stride,
+                    int64_t dst_stride, int dtype, void* stream);
+
+/* The same operators inside the matrix-vector products of a decode step (M = 1..4 bf16 rows, csrc/gemv.hip).
+ * tv_gemv_shift_fwd: y[:, :n1] = hs W[:n1]^T, y[:, n1:] = h W[n1:]^T + bias, with x' / h / hs as tv_norm_shift_fwd
+ *   computes them for one token per sequence (pending, pending_weight: its y and y_weight, or NULL).
+ * tv_gemv_glu_fwd: y = [x | gelu(z) * u] W^T + bias, k1 columns of x; u rows by token id when u_ids.  With a residual
+ *   (M, N) fp32: residual_out = residual + y (fp32) and h_out its bf16 rounding instead of y.                       */
+int tv_gemv_shift_fwd(const float* x, const void* pending, const void* pending_weight, float* x_out, const void* gain,
+                      const void* shift, float* state, const int* start, const int* slot, const void* W, const void* bias,
+                      void* y, int M, int N, int n1, int K, int64_t pending_stride, int64_t state_stride, int64_t ldw,
+                      int64_t y_stride, float eps, void* stream);
+int tv_gemv_glu_fwd(const void* x, const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W,
+                    const void* bias, const float* residual, float* residual_out, void* h_out, void* y, int M, int N, int k1,
+                    int K, int64_t x_stride, int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream);
 
 /* ------------------------------------------------------------------------
  * Linear attention with one constant decay per head, ragged batches:
@@ -558,13 +598,16 @@ int tv_lightning_fwd(const void* q, const void* k, const void* v, const float* d
  * Sequence b: query rows [cu_q[b], cu_q[b+1]); its i-th row sees keys
  * [0, start[b] + i] of key block slot[b] when causal, all start[b] + n_b keys
  * otherwise (start NULL: 0, slot NULL: b).  sink (nheads_q) fp32 or NULL: exp(sink)
- * joins the denominator, unscaled.
+ * joins the denominator, unscaled.  Causal: only keys among the last `window` up to
+ * the query's own or among the first keep_first are seen (INT_MAX, 0: all).  gate or
+ * NULL: o *= sigmoid(gate), rows and heads laid out by its strides.
  * --------------------------------------------------------------------- */
 int tv_attn_generic_fwd(const void* q, const void* k, const void* v, const float* sink, void* o, const int* cu_q,
                         const int* start, const int* slot, int nseq, int64_t rows, int nheads_q, int nheads_kv,
                         int qk_dim, int v_dim, int64_t q_stride_l, int64_t q_stride_h, int64_t k_stride_b,
                         int64_t k_stride_l, int64_t k_stride_h, int64_t v_stride_b, int64_t v_stride_l,
                         int64_t v_stride_h, int64_t o_stride_l, int64_t o_stride_h, float softmax_scale, int causal,
+                        int window, int keep_first, const void* gate, int64_t gate_stride_l, int64_t gate_stride_h,
                         int dtype, void* stream);
 
 /* tv_flash_attn_fwd, causal, with a sink logit per q-head (fp32 or NULL) and a
@@ -575,6 +618,24 @@ int tv_flash_attn_sink_fwd(const void* q, const void* k, const void* v, void* o,
                            int64_t k_stride_l, int64_t k_stride_h, int64_t v_stride_b, int64_t v_stride_l,
                            int64_t v_stride_h, int64_t o_stride_b, int64_t o_stride_l, int64_t o_stride_h,
                            float softmax_scale, int dtype, void* stream);
+
+/* tv_flash_attn_fwd for one sequence (bf16, causal) whose position p sees keys (p - window, p] and the first keep_first
+ * keys; the seqlen_q queries are the last of the seqlen_k positions.  A value dim of its own, optional output gate. */
+int tv_flash_attn_window_fwd(const void* q, const void* k, const void* v, void* o, const void* gate, int window,
+                             int keep_first, int v_dim, int seqlen_q, int seqlen_k, int nheads_q, int nheads_kv, int headdim,
+                             int64_t q_stride_l, int64_t q_stride_h, int64_t k_stride_l, int64_t k_stride_h,
+                             int64_t v_stride_l, int64_t v_stride_h, int64_t o_stride_l, int64_t o_stride_h,
+                             int64_t gate_stride_l, int64_t gate_stride_h, float softmax_scale, int dtype, void* stream);
+
+/* The same attention for one token per sequence (bf16; dims multiples of 8, at most 256): query row b (nheads_q x dim)
+ * against the first keys[b] rows of block slot[b] of cache (slots, capacity, nheads_kv (dim + v_dim)), a row = all keys,
+ * then all values.  fresh (batch, nheads_kv (dim + v_dim)) or NULL: the newest key's row, written to the cache here.   */
+size_t tv_attn_window_decode_workspace_bytes(int batch, int nheads_q, int nheads_kv, int v_dim, int capacity, int window,
+                                             int keep_first);
+int tv_attn_window_decode_fwd(const void* q, void* cache, const void* fresh, const void* gate, void* o, const int* keys,
+                              const int* slot, int batch, int nheads_q, int nheads_kv, int dim, int v_dim, int capacity,
+                              int window, int keep_first, int64_t q_stride, int64_t fresh_stride, int64_t gate_stride,
+                              int64_t o_stride, float scale, void* workspace, size_t workspace_bytes, void* stream);
 
 /* Latent attention of a decode step (bf16, rank a multiple of 8 and <= 512): per
  * sequence b the query row q[b] (nheads x dim) against the first keys[b] rows of

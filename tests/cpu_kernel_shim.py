@@ -7,6 +7,7 @@ import math
 import torch
 
 from oracle import fasovik as OF
+from oracle import fogorax as OG
 from oracle import ops as R
 from oracle import vit as RV
 
@@ -176,7 +177,7 @@ def cpu_kernels():
         "relu2": lambda x, inplace=False: torch.square(torch.relu(x)),
         "causal_conv1d_update": _conv_update, "selective_state_update": _state_update,
         "ssd_state_correction": _state_corr,
-        **POST_NORM_PATCHES,
+        **POST_NORM_PATCHES, **PARALLEL_PATCHES,
     }
     saved = {k: getattr(K, k) for k in patches}
     for k, v in patches.items():
@@ -268,8 +269,74 @@ def _moe_combine(expert_out, pos, weights, residual, norm_weight, eps, weight_of
     return _rms_ex(u, norm_weight, eps, weight_offset, residual=residual, mult=mult, out_dtype=out_dtype)
 
 
+def _embed(ids, table, scale=1.0, positions=None, plan=None):
+    x = table[ids.reshape(-1)].float() * scale
+    if positions is not None:
+        x = x + positions[_places(plan)].float()
+    return x, x.to(table.dtype)
+
+
 POST_NORM_PATCHES = {
-    "embed_scaled": lambda ids, table, scale=1.0: ((table[ids.reshape(-1)].float() * scale), (table[ids.reshape(-1)].float() * scale).to(table.dtype)),
+    "embed_scaled": _embed,
     "rms_norm_ex": _rms_ex, "lightning_attention": _lightning, "attention_sink": _attn_sink, "latent_decode": _latent_decode,
     "moe_router": _moe_router, "moe_plan": _moe_plan, "moe_gemm": _moe_gemm, "moe_combine_norm": _moe_combine,
+}
+
+
+# ------------------------------------------------------------------ parallel layers (oracle/fogorax.py)
+def _places(plan):
+    """the place of every row in its sequence, from the plan's device side"""
+    seq = plan.seq.long()
+    return plan.start.long()[seq] + torch.arange(len(seq)) - plan.cu.long()[seq]
+
+
+def _norm_shift(x, gain, eps, pending=None, pending_weight=None, shift=None, state=None, plan=None, need_h=True):
+    xs = x.double()
+    if pending is not None:
+        xs = xs + OG.rms(pending.double(), eps) * pending_weight.double()
+    h, hs = OG.norm_scalar(xs, gain.double(), eps), None
+    if shift is not None:
+        hs = torch.empty_like(h)
+        for b, s in enumerate(plan.slot.tolist()):
+            lo, hi, st = int(plan.cu[b]), int(plan.cu[b + 1]), int(plan.start[b])
+            before = torch.cat([state[s, (st - 1) & 1].double()[None] if st else torch.zeros_like(h[:1]), h[lo:hi - 1]])
+            hs[lo:hi] = h[lo:hi] + (before - h[lo:hi]) * shift.double()
+            state[s, (st + hi - lo - 1) & 1] = h[hi - 1].float()
+        hs = hs.to(gain.dtype)
+    return (x if pending is None else xs.float()), h.to(gain.dtype), hs
+
+
+def _gated_mul(a, b, act, ids=None, out=None):
+    f = OG.gelu_tanh if act == 1 else OG.sigmoid
+    o = (f(a.double()) * (b if ids is None else b[ids]).double()).to(a.dtype)
+    return o if out is None else out.copy_(o)
+
+
+def _scatter(src, rows, dst):
+    dst[rows.long()] = src
+
+
+def _attn_window(q, cache, plan, kv_heads, scale, window=2 ** 31 - 1, keep_first=0, gate=None, out=None):
+    T, H, d = q.shape
+    e = cache.shape[2] // kv_heads - d
+    o = torch.empty((T, H, e), dtype=q.dtype)
+    for b, s in enumerate(plan.slot.tolist()):
+        lo, hi, st = int(plan.cu[b]), int(plan.cu[b + 1]), int(plan.start[b])
+        k, v = cache[s, :st + hi - lo].double().split([kv_heads * d, kv_heads * e], dim=1)
+        o[lo:hi] = OG.window_attention(q[lo:hi].double(), k.view(-1, kv_heads, d), v.view(-1, kv_heads, e), scale, window, keep_first, start=st).to(q.dtype)
+    if gate is not None:
+        o = (o.double() * OG.sigmoid(gate.double())).to(q.dtype)
+    return o if out is None else out.copy_(o)
+
+
+def _attn_window_decode(q, cache, plan, kv_heads, scale, window=2 ** 31 - 1, keep_first=0, gate=None, fresh=None, out=None):
+    assert plan.decode and plan.keys.tolist() == [a + 1 for a in plan.start.tolist()]
+    if fresh is not None:
+        _scatter(fresh, plan.rows, cache.view(-1, cache.shape[2]))
+    return _attn_window(q, cache, plan, kv_heads, scale, window, keep_first, gate, out)
+
+
+PARALLEL_PATCHES = {
+    "norm_shift": _norm_shift, "residual_add": lambda x, u: (x + u.float(), (x + u.float()).to(u.dtype)), "gated_mul": _gated_mul,
+    "scatter_rows": _scatter, "attention_window": _attn_window, "attention_window_decode": _attn_window_decode,
 }

@@ -56,7 +56,7 @@ def write_folder(path, cfg, tensors):
     (path / "config.json").write_text(json.dumps(cfg))
     header, blobs, at = {}, [], 0
     for name, t in tensors.items():
-        raw = t.contiguous().view(torch.uint8).numpy().tobytes()
+        raw = t.contiguous().flatten().view(torch.uint8).numpy().tobytes()
         header[name] = {"dtype": _NAMES[t.dtype], "shape": list(t.shape), "data_offsets": [at, at + len(raw)]}
         blobs.append(raw)
         at += len(raw)

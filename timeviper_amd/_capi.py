@@ -47,6 +47,9 @@ SIGNATURES = {
     "tv_gemm_set_drip": (None, [_i]),
     "tv_flash_attn_fwd": (_i, [_p] * 5 + [_i] * 6 + [_l] * 12 + [_f, _i, _i, _p]),
     "tv_flash_attn_sink_fwd": (_i, [_p] * 5 + [_i] * 7 + [_l] * 12 + [_f, _i, _p]),
+    "tv_flash_attn_window_fwd": (_i, [_p] * 5 + [_i] * 8 + [_l] * 10 + [_f, _i, _p]),
+    "tv_attn_window_decode_workspace_bytes": (_z, [_i] * 7),
+    "tv_attn_window_decode_fwd": (_i, [_p] * 7 + [_i] * 8 + [_l] * 4 + [_f, _p, _z, _p]),
     "tv_flash_attn_set_variant": (None, [_i]),
     "tv_flash_attn_fp8_workspace_bytes": (_z, [_i] * 5),
     "tv_flash_attn_fp8_fwd": (_i, [_p] * 5 + [_i] * 6 + [_l] * 12 + [_f, _i, _i, _p, _z, _p]),
@@ -69,10 +72,16 @@ SIGNATURES = {
     "tv_patch_embed_fwd": (_i, [_p] * 5 + [_i] * 7 + [_p, _p]),
     "tv_rmsnorm_ex_fwd": (_i, [_p] * 8 + [_l, _l, _i] + [_l] * 5 + [_f] * 3 + [_i] * 3 + [_p]),
     "tv_moe_combine_norm_fwd": (_i, [_p] * 3 + [_i] + [_p] * 4 + [_l, _i] + [_l] * 4 + [_f] * 3 + [_i] * 3 + [_p]),
-    "tv_embed_scaled_fwd": (_i, [_p] * 4 + [_l, _i, _l, _f, _i, _p]),
+    "tv_embed_scaled_fwd": (_i, [_p] * 4 + [_l, _i, _l, _f] + [_p] * 4 + [_l, _i, _p]),
+    "tv_norm_shift_fwd": (_i, [_p] * 13 + [_l, _i, _l, _l, _f, _i, _p]),
+    "tv_residual_add_fwd": (_i, [_p] * 4 + [_l, _i, _l, _i, _p]),
+    "tv_gated_mul_fwd": (_i, [_p] * 4 + [_l, _i] + [_l] * 4 + [_i, _i, _p]),
+    "tv_scatter_rows": (_i, [_p] * 3 + [_l, _i, _l, _l, _i, _p]),
+    "tv_gemv_shift_fwd": (_i, [_p] * 12 + [_i] * 4 + [_l] * 4 + [_f, _p]),
+    "tv_gemv_glu_fwd": (_i, [_p] * 4 + [_l] + [_p] * 6 + [_i] * 4 + [_l] * 5 + [_p]),
     "tv_lightning_workspace_bytes": (_z, [_i] * 6),
     "tv_lightning_fwd": (_i, [_p] * 8 + [_i, _i, _p, _z] + [_i] * 3 + [_l] * 4 + [_i, _i, _p]),
-    "tv_attn_generic_fwd": (_i, [_p] * 8 + [_i, _l] + [_i] * 4 + [_l] * 10 + [_f, _i, _i, _p]),
+    "tv_attn_generic_fwd": (_i, [_p] * 8 + [_i, _l] + [_i] * 4 + [_l] * 10 + [_f] + [_i] * 3 + [_p, _l, _l, _i, _p]),
     "tv_latent_query_fwd": (_i, [_p] * 3 + [_i] * 4 + [_l] * 3 + [_i, _p]),
     "tv_latent_value_fwd": (_i, [_p] * 3 + [_i] * 4 + [_l] * 3 + [_i, _p]),
     "tv_latent_decode_workspace_bytes": (_z, [_i] * 4),
@@ -90,7 +99,7 @@ class TimeViperHipError(RuntimeError):
     pass
 
 
-ABI_VERSION = 13      # tv_abi_version() of the library these SIGNATURES describe (csrc/capi.cpp)
+ABI_VERSION = 14      # tv_abi_version() of the library these SIGNATURES describe (csrc/capi.cpp)
 
 
 def lib_path() -> Path:

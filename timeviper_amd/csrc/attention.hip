@@ -82,6 +82,9 @@ struct AttnArgs {
   int o16;           // streaming kernel: o rows are 16-byte aligned (wide epilogue stores)
   int Dv;            // value head dim (D unless the caller says otherwise)
   const float* sink; // per q-head logit without key or value that joins the denominator, or NULL (flash_fwd_kernel, causal)
+  int window, keep;  // flash_fwd_kernel with WIN: position p sees keys (p - window, p] and the first `keep`
+  const void* gate;  // WIN: o is multiplied by sigmoid(gate), element by element, or NULL
+  int64_t gsl, gsh;
   int notrim;        // streaming kernel (dev, TV_FA_TRIM=0): the last key tile runs all its sub-tiles
 };
 
@@ -93,7 +96,9 @@ struct AttnArgs {
 // XOR-swizzled on the DMA source address so that the row reads of K (ds_read_b128, chunk ^
 // row%16) and the transposing reads of V (ds_read_b64_tr_b16, chunk ^ 4(row%4)) are bank
 // conflict free.  Chunks past head_dim are never copied (the K ones QK^T reads are zeroed once).
-template <typename T, int KS, int DT, int NW, int KT>
+// WIN: causal with a sliding window and kept first keys.  The work-group visits the tiles that hold kept keys, then jumps to the
+// first tile of its first row's window: ring, copies and waits count the visited tiles.
+template <typename T, int KS, int DT, int NW, int KT, bool WIN = false>
 __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
   constexpr int FA_KB = 32 * KT;     // keys per tile
   constexpr int NPK = FA_KB / 4;     // 1 KiB DMA pieces (4 key rows) of K per tile; as many of V
@@ -175,7 +180,14 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
   const int wg_q_last = min(qblk * QB + QB, a.Lq) - 1;
   int k_end = a.causal ? min(a.Lk, wg_q_last + shift + 1) : a.Lk;
   if (k_end < 0) k_end = 0;
-  const int ntiles = (k_end + FA_KB - 1) / FA_KB;
+  int ntiles = (k_end + FA_KB - 1) / FA_KB;
+  int tkeep = 0, tskip = 0;                     // WIN: visited tile i is tile i, or i + tskip from tkeep on
+  if constexpr (WIN) {
+    tkeep = (min(a.keep, k_end) + FA_KB - 1) / FA_KB;
+    tskip = max(max(0, qblk * QB + shift - a.window + 1) / FA_KB - tkeep, 0);
+    ntiles -= tskip;
+  }
+  auto key_of_tile = [&](int kt) __attribute__((always_inline)) { return (WIN && kt >= tkeep ? kt + tskip : kt) * FA_KB; };
 
   // ---- DMA pieces of this wave: piece id pc = wave + NW*i; pc < 16 -> K rows 4pc..4pc+3,
   // else V rows 4(pc-16)..; lane l carries row 4(pc%16) + l/16, LDS slot l%16 ----
@@ -193,7 +205,7 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
     p_off[i] = (unsigned)(((int64_t)row * (isK ? a.ksl : a.vsl) + c * 8) * (int)sizeof(T));
   }
   auto issue_piece = [&](int kt, int i) {          // piece i (0..PPW-1) of tile kt
-    const int kbase = kt * FA_KB;
+    const int kbase = key_of_tile(kt);
     const int stage = kt % NS;
     const int pc = wave + NW * i;
     const bool isK = pc < NPK;           // wave-uniform
@@ -241,7 +253,7 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
   }
 
   for (int kt = 0; kt < ntiles; ++kt) {
-    const int kbase = kt * FA_KB;
+    const int kbase = key_of_tile(kt);
     const bool ahead = kt + 2 < ntiles;
     // stage bases as LDS byte offsets (scalar), folded into one base register per fragment family
     const unsigned stage_off = (unsigned)((kt % NS) * TILEB);
@@ -249,7 +261,8 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
 
     // wave-uniform skip of tiles entirely above this wave's causal diagonal
     const int wave_q_last = q0 + FA_QW - 1;
-    const bool active = !(a.causal && kbase > wave_q_last + shift);
+    bool active = !(a.causal && kbase > wave_q_last + shift);
+    if constexpr (WIN) active = active && (kbase < a.keep || kbase + FA_KB > q0 + shift - a.window + 1);
     if (!active && ahead) issue_tile(kt + 2);
     if (active) {
       // ---- S^T = K . Q^T  (2 key sub-tiles of 32); all K fragment reads ahead of the MFMAs;
@@ -284,14 +297,16 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
       // ---- mask, running max on the raw scores (the scale is positive, so it commutes with
       // max), then p = 2^(s*scale - m) as one FMA + v_exp per score; packed fp32 math ----
       typedef float f32x2 __attribute__((ext_vector_type(2)));
-      const bool need_mask = (kbase + FA_KB > a.Lk) || (a.causal && kbase + FA_KB - 1 > q0 + shift);
+      bool need_mask = (kbase + FA_KB > a.Lk) || (a.causal && kbase + FA_KB - 1 > q0 + shift);
+      if constexpr (WIN) need_mask = need_mask || (kbase <= wave_q_last + shift - a.window && kbase + FA_KB > a.keep);
       if (need_mask) {
 #pragma unroll
         for (int t = 0; t < KT; ++t)
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = kbase + t * 32 + (i & 3) + 8 * (i >> 2) + 4 * hh;
-            const bool ok = key < a.Lk && (!a.causal || key <= qrow + shift);
+            bool ok = key < a.Lk && (!a.causal || key <= qrow + shift);
+            if constexpr (WIN) ok = ok && (key > qrow + shift - a.window || key < a.keep);
             sacc[t][i] = ok ? sacc[t][i] : -INFINITY;
           }
       }
@@ -386,6 +401,13 @@ __global__ __launch_bounds__(NW * 64) void flash_fwd_kernel(AttnArgs a) {
         const int d0 = dt * 32 + 8 * g + 4 * hh;
         if (d0 < a.Dv) {
           v4 pk;
+          if constexpr (WIN) {
+            if (a.gate) {
+              const v4 gt = *(const v4*)((const T*)a.gate + (int64_t)qrow * a.gsl + (int64_t)h * a.gsh + d0);
+#pragma unroll
+              for (int j = 0; j < 4; ++j) oacc[dt][4 * g + j] *= sigmoid_f((float)gt[j]);
+            }
+          }
 #pragma unroll
           for (int j = 0; j < 4; ++j) pk[j] = from_f32<T>(oacc[dt][4 * g + j] * inv);
           *(v4*)(op + d0) = pk;
@@ -895,9 +917,33 @@ int launch_fa_d(const AttnArgs& a, int B, hipStream_t st) {
   TV_LAUNCH_CHECK();
 }
 
+// windowed form: bf16, one query block of 256 (or, for short portions, 128) rows a work-group; 64-key tiles at head dim 128
+// (the bounds of the window do not fit beside 96 keys' fragments)
+template <int KS, int DT>
+int launch_fa_win(const AttnArgs& a, int B, hipStream_t st) {
+  constexpr int KT = KS > 6 ? 2 : FA_KT, lds = 2 * 3 * 32 * KT * 256;
+  const bool big = a.Lq > 128;
+  const void* f = big ? (const void*)flash_fwd_kernel<bf16_t, KS, DT, 8, KT, true> : (const void*)flash_fwd_kernel<bf16_t, KS, DT, 4, KT, true>;
+  const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  if (e != hipSuccess) {
+    tv_set_error("flash_attn: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+    return TV_ERR_LAUNCH;
+  }
+  if (big) flash_fwd_kernel<bf16_t, KS, DT, 8, KT, true><<<dim3((a.Lq + 255) / 256, a.Hq, B), 512, lds, st>>>(a);
+  else flash_fwd_kernel<bf16_t, KS, DT, 4, KT, true><<<dim3((a.Lq + 127) / 128, a.Hq, B), 256, lds, st>>>(a);
+  TV_LAUNCH_CHECK();
+}
+
 template <typename T>
 int launch_fa(const AttnArgs& a, int B, hipStream_t st) {
   const int D = a.D > a.Dv ? a.D : a.Dv;
+  if constexpr (std::is_same<T, bf16_t>::value) {
+    if (a.window > 0) {
+      if (D <= 64) return launch_fa_win<4, 2>(a, B, st);
+      if (D <= 96) return launch_fa_win<6, 3>(a, B, st);
+      if (D <= 128) return launch_fa_win<8, 4>(a, B, st);
+    }
+  }
   if (D <= 64) return launch_fa_d<T, 4, 2>(a, B, st);
   if (D <= 80) return launch_fa_d<T, 5, 3>(a, B, st);
   if (D <= 96) return launch_fa_d<T, 6, 3>(a, B, st);
@@ -915,7 +961,13 @@ extern "C" int tv_fa_debug_stamps(unsigned long long* out) {
 
 extern "C" void tv_flash_attn_set_variant(int variant) { g_fa_variant.store(variant, std::memory_order_relaxed); }
 
-static int flash_fwd(const void* q, const void* k, const void* v, void* o, void* lse, const float* sink, int v_dim,
+struct FlashWindow {
+  int window = 0, keep = 0;      // window 0: every key up to the query's own position
+  const void* gate = nullptr;
+  int64_t gsl = 0, gsh = 0;
+};
+
+static int flash_fwd(const FlashWindow& win, const void* q, const void* k, const void* v, void* o, void* lse, const float* sink, int v_dim,
                                  int batch, int seqlen_q, int seqlen_k, int nheads_q,
                                  int nheads_kv, int headdim, int64_t q_stride_b,
                                  int64_t q_stride_l, int64_t q_stride_h, int64_t k_stride_b,
@@ -955,6 +1007,7 @@ static int flash_fwd(const void* q, const void* k, const void* v, void* o, void*
   a.nb = batch;
   a.Dv = v_dim;
   a.sink = sink;
+  a.window = win.window; a.keep = win.keep; a.gate = win.gate; a.gsl = win.gsl; a.gsh = win.gsh;
   hipStream_t st = (hipStream_t)stream;
   if (dtype == TV_BF16) return launch_fa<bf16_t>(a, batch, st);
   return launch_fa<f16_t>(a, batch, st);
@@ -968,7 +1021,7 @@ extern "C" int tv_flash_attn_fwd(const void* q, const void* k, const void* v, vo
                                  int64_t v_stride_l, int64_t v_stride_h, int64_t o_stride_b,
                                  int64_t o_stride_l, int64_t o_stride_h, float softmax_scale,
                                  int causal, int dtype, void* stream) {
-  return flash_fwd(q, k, v, o, lse, nullptr, headdim, batch, seqlen_q, seqlen_k, nheads_q, nheads_kv, headdim, q_stride_b, q_stride_l,
+  return flash_fwd(FlashWindow{}, q, k, v, o, lse, nullptr, headdim, batch, seqlen_q, seqlen_k, nheads_q, nheads_kv, headdim, q_stride_b, q_stride_l,
                    q_stride_h, k_stride_b, k_stride_l, k_stride_h, v_stride_b, v_stride_l, v_stride_h, o_stride_b, o_stride_l, o_stride_h,
                    softmax_scale, causal, dtype, stream);
 }
@@ -982,7 +1035,25 @@ extern "C" int tv_flash_attn_sink_fwd(const void* q, const void* k, const void* 
                                  int64_t v_stride_l, int64_t v_stride_h, int64_t o_stride_b,
                                  int64_t o_stride_l, int64_t o_stride_h, float softmax_scale,
                                  int dtype, void* stream) {
-  return flash_fwd(q, k, v, o, nullptr, sink, v_dim, batch, seqlen_q, seqlen_k, nheads_q, nheads_kv, headdim, q_stride_b, q_stride_l,
+  return flash_fwd(FlashWindow{}, q, k, v, o, nullptr, sink, v_dim, batch, seqlen_q, seqlen_k, nheads_q, nheads_kv, headdim, q_stride_b, q_stride_l,
                    q_stride_h, k_stride_b, k_stride_l, k_stride_h, v_stride_b, v_stride_l, v_stride_h, o_stride_b, o_stride_l, o_stride_h,
                    softmax_scale, 1, dtype, stream);
+}
+
+// Causal attention of one sequence with a sliding window and kept first keys, a value dim of its own and an optional output gate
+// (o *= sigmoid(gate)); bf16.
+extern "C" int tv_flash_attn_window_fwd(const void* q, const void* k, const void* v, void* o, const void* gate, int window,
+                                        int keep_first, int v_dim, int seqlen_q, int seqlen_k, int nheads_q, int nheads_kv, int headdim,
+                                        int64_t q_stride_l, int64_t q_stride_h, int64_t k_stride_l, int64_t k_stride_h,
+                                        int64_t v_stride_l, int64_t v_stride_h, int64_t o_stride_l, int64_t o_stride_h,
+                                        int64_t gate_stride_l, int64_t gate_stride_h, float softmax_scale, int dtype, void* stream) {
+  TV_CHECK_ARG(window > 0 && keep_first >= 0 && seqlen_k >= seqlen_q, "flash_attn_window: bad window or lengths");
+  if (dtype != TV_BF16) TV_UNSUPPORTED("flash_attn_window: dtype must be bf16");
+  if (headdim > 128 || v_dim > 128) TV_UNSUPPORTED("flash_attn_window: headdim %d / %d > 128", headdim, v_dim);
+  if (gate && (gate_stride_l % 4 || gate_stride_h % 4 || ((uintptr_t)gate & 7)))
+    TV_UNSUPPORTED("flash_attn_window: gate rows must be 8-byte aligned");
+  FlashWindow w;
+  w.window = window; w.keep = keep_first; w.gate = gate; w.gsl = gate_stride_l; w.gsh = gate_stride_h;
+  return flash_fwd(w, q, k, v, o, nullptr, nullptr, v_dim, 1, seqlen_q, seqlen_k, nheads_q, nheads_kv, headdim, 0, q_stride_l, q_stride_h,
+                   0, k_stride_l, k_stride_h, 0, v_stride_l, v_stride_h, 0, o_stride_l, o_stride_h, softmax_scale, 1, dtype, stream);
 }

@@ -7,6 +7,8 @@
 // Sequence b owns query rows [cu_q[b], cu_q[b + 1]); its keys are rows [0, start[b] + i] of key block slot[b] for its i-th
 // query row when causal (start: the tokens that were there before), all start[b] + n_b keys otherwise.
 // A sink is a learned logit without key or value: exp(sink_h) is one more term of the denominator, not scaled.
+// Causal with a window: position p sees keys (p - window, p] and the first `keep` keys of its sequence; the loop runs over the
+// visible keys only.  gate: the output is multiplied by sigmoid(gate), element by element.
 #include "common.hpp"
 
 namespace {
@@ -19,9 +21,11 @@ struct AgArgs {
   const float* sink;
   void* o;
   const int *cu_q, *start, *slot;
-  int nseq, H, gq, dk, dv, causal;
+  int nseq, H, gq, dk, dv, causal, window, keep;
   int64_t qsl, qsh, ksb, ksl, ksh, vsb, vsl, vsh, osl, osh;
   float scale;
+  const void* gate;
+  int64_t gsl, gsh;
 };
 
 template <typename T>
@@ -36,7 +40,9 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(AgArgs a) {
   int b = 0;
   while (b + 1 < a.nseq && row >= a.cu_q[b + 1]) ++b;
   const int n_b = a.cu_q[b + 1] - a.cu_q[b], i = row - a.cu_q[b], st = a.start ? a.start[b] : 0;
-  const int nk = a.causal ? st + i + 1 : st + n_b;
+  const int end = a.causal ? st + i + 1 : st + n_b;
+  const int lo = a.causal ? max(0, end - a.window) : 0, kept = min(a.keep, lo);      // keys [0, kept) and [lo, end)
+  const int nk = kept + end - lo, skip = lo - kept;                                  // visible key j: j, or j + skip from kept on
   const int64_t blk = a.slot ? a.slot[b] : b;
   const T* kb = (const T*)a.k + blk * a.ksb + (int64_t)(h / a.gq) * a.ksh;
   const T* vb = (const T*)a.v + blk * a.vsb + (int64_t)(h / a.gq) * a.vsh;
@@ -56,7 +62,7 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(AgArgs a) {
     const int key = k0 + tid;
     float s = -INFINITY;
     if (key < nk) {
-      const T* kr = kb + (int64_t)key * a.ksl;
+      const T* kr = kb + (int64_t)(key < kept ? key : key + skip) * a.ksl;
       float dot = 0.f;
       for (int d = 0; d < a.dk; ++d) dot = fmaf(sq[d], to_f32(kr[d]), dot);
       s = dot * a.scale;
@@ -84,7 +90,7 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(AgArgs a) {
     const int kn = min(AG_THREADS, nk - k0);
     for (int kk = grp; kk < kn; kk += ng) {
       const float pk = sp[kk];
-      const T* vr = vb + (int64_t)(k0 + kk) * a.vsl;
+      const T* vr = vb + (int64_t)(k0 + kk < kept ? k0 + kk : k0 + kk + skip) * a.vsl;
 #pragma unroll
       for (int j = 0; j < AG_MAXNV; ++j) {
         const int d = vd + j * wid;
@@ -104,7 +110,11 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(AgArgs a) {
         float t = 0.f;
         for (int g = 0; g < ng; ++g) t += sacc[g * wid + vd];
         const int d = vd + j * wid;
-        if (d < a.dv) orow[d] = from_f32<T>(t * inv);
+        if (d < a.dv) {
+          t *= inv;
+          if (a.gate) t *= sigmoid_f(to_f32(((const T*)a.gate)[(int64_t)row * a.gsl + (int64_t)h * a.gsh + d]));
+          orow[d] = from_f32<T>(t);
+        }
       }
       __syncthreads();
     }
@@ -118,16 +128,17 @@ extern "C" int tv_attn_generic_fwd(const void* q, const void* k, const void* v, 
                                    int qk_dim, int v_dim, int64_t q_stride_l, int64_t q_stride_h, int64_t k_stride_b,
                                    int64_t k_stride_l, int64_t k_stride_h, int64_t v_stride_b, int64_t v_stride_l,
                                    int64_t v_stride_h, int64_t o_stride_l, int64_t o_stride_h, float softmax_scale, int causal,
+                                   int window, int keep_first, const void* gate, int64_t gate_stride_l, int64_t gate_stride_h,
                                    int dtype, void* stream) {
   TV_CHECK_ARG(nseq > 0 && rows >= 0 && rows < (1ll << 31) && nheads_q > 0 && nheads_kv > 0 && nheads_q % nheads_kv == 0 &&
-                   qk_dim > 0 && v_dim > 0, "attn_generic: bad sizes");
+                   qk_dim > 0 && v_dim > 0 && window > 0 && keep_first >= 0, "attn_generic: bad sizes");
   if (rows == 0) return TV_OK;
   TV_CHECK_ARG(q && k && v && o && cu_q, "attn_generic: null pointer");
   if (dtype != TV_F32 && dtype != TV_BF16) TV_UNSUPPORTED("attn_generic: dtype must be fp32 or bf16");
   if (v_dim > AG_THREADS * AG_MAXNV || qk_dim > 4096) TV_UNSUPPORTED("attn_generic: qk_dim %d / v_dim %d", qk_dim, v_dim);
-  AgArgs a{q, k, v, sink, o, cu_q, start, slot, nseq, nheads_q, nheads_q / nheads_kv, qk_dim, v_dim, causal,
+  AgArgs a{q, k, v, sink, o, cu_q, start, slot, nseq, nheads_q, nheads_q / nheads_kv, qk_dim, v_dim, causal, window, keep_first,
            q_stride_l, q_stride_h, k_stride_b, k_stride_l, k_stride_h, v_stride_b, v_stride_l, v_stride_h, o_stride_l, o_stride_h,
-           softmax_scale};
+           softmax_scale, gate, gate_stride_l, gate_stride_h};
   const size_t lds = ((qk_dim + 3) / 4 * 4 + 2 * AG_THREADS) * sizeof(float);
   const dim3 grid((unsigned)rows, (unsigned)nheads_q);
   if (dtype == TV_F32) attn_generic_kernel<float><<<grid, AG_THREADS, lds, (hipStream_t)stream>>>(a);

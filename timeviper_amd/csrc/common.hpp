@@ -28,6 +28,11 @@ template <typename T> __device__ __forceinline__ float to_f32(T v) { return (flo
 template <typename T> __device__ __forceinline__ T from_f32(float v) { return (T)v; }
 
 __device__ __forceinline__ float silu_f(float x) { return x / (1.f + __expf(-x)); }
+__device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + __expf(-x)); }
+// 0.5 x (1 + tanh(u)) = x sigmoid(2 u), u = sqrt(2 / pi) (x + 0.044715 x^3)
+__device__ __forceinline__ float gelu_tanh_f(float x) {
+  return x * sigmoid_f(1.5957691216057308f * fmaf(0.044715f * x * x, x, x));
+}
 // softplus with torch's default threshold (20): identical branch to
 // F.softplus and to upstream's `dt < 20` guard.
 __device__ __forceinline__ float softplus_f(float x) {

@@ -17,14 +17,19 @@
 //   PRO_POSTNORM  x' = residual + mult * (x * rsqrt(mean(x^2) + eps)) * (w_offset + w), fp32 (written to `res_out`, its bf16
 //                 rounding to `h_out`, by work-group 0), f = bf16(x')    post-norm models: the norm of the sublayer in front
 //   PRO_NORMGATE  f = bf16(x * rsqrt(mean(x^2) + eps) * w * sigmoid(gate))     lightning attention's output norm and gate
-// (the last two belong to models on a 32-bit residual stream and agree with tv_rmsnorm_ex_fwd)
+//   PRO_SHIFT     x' = residual + rms(x) * w (the norm of what waits, optional; fp32, to `res_out`), h = rms(x') * gain,
+//                 hs = h + (h_before - h) * shift with the h of the sequence's previous token from its state (the new one goes to
+//                 the state's other row): rows of W below N1 meet bf16(hs), the others bf16(h) and a bias
+//   PRO_GLU       f = [x | bf16(gelu_tanh(z) * u)]: columns below K1 are x, the others a gated product, u's rows optionally
+//                 gathered by token id; epilogue: y + bias + residual in fp32 (`res_out`, `h_out`) when there is a residual
+// (the last four belong to models on a 32-bit residual stream and agree with tv_rmsnorm_ex_fwd, tv_norm_shift_fwd and tv_gated_mul_fwd)
 // with the rounding points of the stand-alone kernels (norms.hip), so the fused step and the unfused one agree to the
 // accumulation order of the dot products.  fp32 accumulation (v_dot2c_f32_bf16), one rounding of y.
 #include "ssd_common.hpp"
 
 namespace {
 
-enum { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_RELU2 = 2, PRO_GATED = 3, PRO_POSTNORM = 4, PRO_NORMGATE = 5 };
+enum { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_RELU2 = 2, PRO_GATED = 3, PRO_POSTNORM = 4, PRO_NORMGATE = 5, PRO_SHIFT = 6, PRO_GLU = 7 };
 constexpr int GV_THREADS = 256;
 constexpr int GV_WAVES = GV_THREADS / 64;
 constexpr int GV_MAXM = 4;
@@ -47,6 +52,17 @@ struct GemvArgs {
   float* res_out;
   bf16_t* h_out;
   float mult, woff;
+  // PRO_SHIFT: x waits in `delta` (or NULL), its norm weight in norm_w (bf16); rows of W below N1 meet hs
+  const bf16_t *gain, *shift;
+  float* state;                    // blocks of (2, K), `sst` floats apart; row p & 1: the h of position p
+  const int *start, *slot;
+  int64_t sst;
+  int N1;
+  // PRO_GLU
+  int K1;
+  const bf16_t *z, *u;
+  const int64_t* u_ids;
+  int64_t zs, us, u_rows;
 };
 
 // the 8 norm weights of one 16-byte piece of x: requested here (fp32 weights: two 16-byte loads, bf16: one), turned into
@@ -220,6 +236,111 @@ __device__ __forceinline__ void gemv_prologue(const GemvArgs& a, bf16_t* fx, flo
           }
         }
       }
+    } else if (PRO == PRO_SHIFT) {
+      constexpr int MAXV = 4;                        // K <= 8 * 256 * 4 (launcher)
+      const int st = a.start[m];
+      float* sr = a.state + (int64_t)a.slot[m] * a.sst;
+      const float *rr = a.res + (int64_t)m * K, *pr = sr + (int64_t)((st - 1) & 1) * K;
+      bf16x8 dq[MAXV], wq[MAXV], hq[MAXV];
+      f32x4 r0[MAXV], r1[MAXV], p0[MAXV], p1[MAXV];
+#pragma unroll
+      for (int k = 0; k < MAXV; ++k) {               // (lanes past the end request the last piece again: no branch around a load)
+        if (k * GV_THREADS >= nv) break;
+        const int iv = min(tid + k * GV_THREADS, nv - 1);
+        r0[k] = *(const f32x4*)(rr + 8 * iv);
+        r1[k] = *(const f32x4*)(rr + 8 * iv + 4);
+        if (a.delta) {
+          dq[k] = *(const bf16x8*)(a.delta + (int64_t)m * a.ds + 8 * iv);
+          wq[k] = *(const bf16x8*)((const bf16_t*)a.norm_w + 8 * iv);
+        }
+        hq[k] = *(const bf16x8*)(a.shift + 8 * iv);
+        p0[k] = *(const f32x4*)(pr + 8 * iv);
+        p1[k] = *(const f32x4*)(pr + 8 * iv + 4);
+      }
+      const float gain = (float)*a.gain;
+      __builtin_amdgcn_sched_barrier(0);
+      if (m == 0) after_loads();
+      __builtin_amdgcn_sched_barrier(0);
+      auto total = [&](float v) __attribute__((always_inline)) {
+        v = wave_sum(v);
+        __syncthreads();                             // (red is used again)
+        if (lane == 0) red[wave] = v;
+        __syncthreads();
+        float t = 0.f;
+#pragma unroll
+        for (int i = 0; i < GV_WAVES; ++i) t += red[i];
+        return t;
+      };
+      if (a.delta) {
+        float ssq = 0.f;
+#pragma unroll
+        for (int k = 0; k < MAXV; ++k)
+          if (tid + k * GV_THREADS < nv) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) ssq = fmaf((float)dq[k][j], (float)dq[k][j], ssq);
+          }
+        const float rstd = rsqrtf(total(ssq) / (float)K + a.eps);
+#pragma unroll
+        for (int k = 0; k < MAXV; ++k) {
+          const int iv = tid + k * GV_THREADS;
+          if (iv < nv) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+              r0[k][j] = fmaf((float)dq[k][j] * rstd, (float)wq[k][j], r0[k][j]);
+              r1[k][j] = fmaf((float)dq[k][4 + j] * rstd, (float)wq[k][4 + j], r1[k][j]);
+            }
+            if (blockIdx.x == 0) {
+              float* ro = a.res_out + (int64_t)m * K + 8 * iv;
+              *(f32x4*)ro = r0[k];
+              *(f32x4*)(ro + 4) = r1[k];
+            }
+          }
+        }
+      }
+      float ssq = 0.f;
+#pragma unroll
+      for (int k = 0; k < MAXV; ++k)
+        if (tid + k * GV_THREADS < nv) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) ssq = fmaf(r0[k][j], r0[k][j], fmaf(r1[k][j], r1[k][j], ssq));
+        }
+      const float rstd = rsqrtf(total(ssq) / (float)K + a.eps) * gain;
+      bf16_t* fh = fx + (int64_t)(a.M + m) * K;
+#pragma unroll
+      for (int k = 0; k < MAXV; ++k) {
+        const int iv = tid + k * GV_THREADS;
+        if (iv < nv) {
+          bf16x8 o, os;
+          r0[k] *= rstd;
+          r1[k] *= rstd;
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const float h = j < 4 ? r0[k][j & 3] : r1[k][j & 3], before = st > 0 ? (j < 4 ? p0[k][j & 3] : p1[k][j & 3]) : 0.f;
+            o[j] = (bf16_t)h;
+            os[j] = (bf16_t)fmaf(before - h, (float)hq[k][j], h);
+          }
+          *(bf16x8*)(fr + 8 * iv) = os;
+          *(bf16x8*)(fh + 8 * iv) = o;
+          if (blockIdx.x == 0) {                     // (the other row of the state: nobody reads it in this launch)
+            float* so = sr + (int64_t)(st & 1) * K + 8 * iv;
+            *(f32x4*)so = r0[k];
+            *(f32x4*)(so + 4) = r1[k];
+          }
+        }
+      }
+    } else if (PRO == PRO_GLU) {
+      if (m == 0) after_loads();
+      const int nv1 = a.K1 / 8;
+      for (int iv = tid; iv < nv1; iv += GV_THREADS) *(bf16x8*)(fr + 8 * iv) = *(const bf16x8*)(xr + 8 * iv);
+      const int64_t ur = a.u_ids ? a.u_ids[m] : m;
+      const bool ok = ur >= 0 && ur < a.u_rows;      // (callers check ids on the host; a bad one reads nothing)
+      for (int iv = tid; iv < nv - nv1; iv += GV_THREADS) {
+        const bf16x8 z = *(const bf16x8*)(a.z + (int64_t)m * a.zs + 8 * iv), zero = {};
+        bf16x8 u = ok ? *(const bf16x8*)(a.u + ur * a.us + 8 * iv) : zero;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) u[j] = (bf16_t)(gelu_tanh_f((float)z[j]) * (float)u[j]);
+        *(bf16x8*)(fr + 8 * (nv1 + iv)) = u;
+      }
     } else {                                         // PRO_GATED: a wave per group of `group` channels
       constexpr int MAXV = 4, GPW = 1;               // group <= 8 * 64 * 4 (launcher)
       const int ngroups = K / a.group, gv = a.group / 8;
@@ -382,7 +503,11 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_bf16_kernel(GemvArgs a) {
           float sm = 0.f;
 #pragma unroll
           for (int w = 0; w < GV_WAVES; ++w) sm += part[par][j][w][r][m];
-          if (a.y32) a.y32[(int64_t)m * a.ys + n] = sm;
+          if (PRO == PRO_GLU && a.res) {
+            const float v = sm + (a.bias ? (float)a.bias[n] : 0.f) + a.res[(int64_t)m * a.N + n];
+            a.res_out[(int64_t)m * a.N + n] = v;
+            if (a.h_out) a.h_out[(int64_t)m * a.N + n] = (bf16_t)v;
+          } else if (a.y32) a.y32[(int64_t)m * a.ys + n] = sm;
           else a.y[(int64_t)m * a.ys + n] = (bf16_t)(sm + (a.bias ? (float)a.bias[n] : 0.f));
         }
       }
@@ -442,10 +567,16 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
 #pragma unroll
           for (int m = 0; m < MT; ++m)
             if (MT == 1 || m < a.M) {
-              const bf16x8 xv = *(const bf16x8*)(fl + (int64_t)m * K + 512 * (i0 + u));
+              // (PRO_SHIFT: hs for the rows below N1, h — behind it in LDS — for the others)
+              const int o0 = PRO == PRO_SHIFT && n0 >= a.N1 ? a.M * K : 0;
+              const bf16x8 xv = *(const bf16x8*)(fl + o0 + (int64_t)m * K + 512 * (i0 + u));
 #pragma unroll
               for (int r = 0; r < R; ++r)
-                if (n0 + r * TW < a.N) acc[r][m] = dot8(w[u][r], xv, acc[r][m]);
+                if (n0 + r * TW < a.N) {
+                  if (PRO == PRO_SHIFT && o0 == 0 && n0 + r * TW >= a.N1)      // (wave uniform)
+                    acc[r][m] = dot8(w[u][r], *(const bf16x8*)(fl + (int64_t)(a.M + m) * K + 512 * (i0 + u)), acc[r][m]);
+                  else acc[r][m] = dot8(w[u][r], xv, acc[r][m]);
+                }
             }
         }
     };
@@ -472,7 +603,8 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
 #pragma unroll
       for (int m = 0; m < MT; ++m) tot[r][m] = (MT == 1 || m < a.M) ? wave_total(acc[r][m]) : 0.f;
     if (lane < R && nmine < a.N) {
-      const float bs = a.bias ? (float)a.bias[nmine] : 0.f;
+      const int nb = PRO == PRO_SHIFT ? nmine - a.N1 : nmine;        // (PRO_SHIFT: the bias belongs to the rows from N1 on)
+      const float bs = a.bias && nb >= 0 ? (float)a.bias[nb] : 0.f;
 #pragma unroll
       for (int m = 0; m < MT; ++m)
         if (MT == 1 || m < a.M) {
@@ -497,14 +629,18 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
             *(bf16x4*)st = win;
             out = (bf16_t)silu_f(acc_c);
           }
-          if (a.y32) a.y32[(int64_t)m * a.ys + nmine] = v;
+          if (PRO == PRO_GLU && a.res) {
+            v += bs + a.res[(int64_t)m * a.N + nmine];
+            a.res_out[(int64_t)m * a.N + nmine] = v;
+            if (a.h_out) a.h_out[(int64_t)m * a.N + nmine] = (bf16_t)v;
+          } else if (a.y32) a.y32[(int64_t)m * a.ys + nmine] = v;
           else a.y[(int64_t)m * a.ys + nmine] = out;
         }
     }
   }
 }
 
-// ---------------------------------------------------------------- round 6: one row of x, split-K, f(x) in registers
+// ---------------------------------------------------------------- one row of x, split-K, f(x) in registers
 // The split-K kernel above stages f(x) in LDS behind a barrier: 1.5 - 3 us in front of the first product of a work-group
 // that streams 160 - 280 KB in 16 - 24 us.  With one row of x a wave needs only ITS quarter of f(x) (5 - 8 pieces of 16
 // bytes a lane: 20 - 32 registers), so it can hold it itself and start its products as soon as its own operands are
@@ -672,7 +808,7 @@ int launch_gemv_r(const GemvArgs& a, hipStream_t st) {
 }
 template <int PRO, int MT, bool NT, int R, int NB>
 int launch_gemv_rows(const GemvArgs& a, hipStream_t st) {
-  const size_t lds = (size_t)a.M * a.K * sizeof(bf16_t);
+  const size_t lds = (size_t)(PRO == PRO_SHIFT ? 2 : 1) * a.M * a.K * sizeof(bf16_t);
   static const hipError_t attr = hipFuncSetAttribute((const void*)gemv_rows_kernel<PRO, MT, NT, R, NB>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
   if (attr != hipSuccess) {
@@ -715,6 +851,7 @@ int launch_gemv_m(const GemvArgs& a, hipStream_t st) {
   }
   // (the gated prologue holds two groups' operands in registers: no second set of W rows beside them)
   constexpr bool PF = PRO != PRO_GATED;
+  if constexpr (PRO == PRO_SHIFT) return gemv_nt() ? launch_gemv_rows<PRO, MT, true, 2, 10>(a, st) : launch_gemv_rows<PRO, MT, false, 2, 10>(a, st);
   if (!gemv_nt()) return splitk ? launch_gemv_r<PRO, MT, 2, 8, false, PF>(a, st) : launch_gemv_rows<PRO, MT, false, 2, 10>(a, st);
   return splitk ? launch_gemv_r<PRO, MT, 2, 8, true, PF>(a, st) : launch_gemv_rows<PRO, MT, true, 2, 10>(a, st);
 }
@@ -805,4 +942,45 @@ extern "C" int tv_gemv_post_fwd(const void* x, const void* W, void* y, int y_dty
   TV_CHECK_ARG(gate, "gemv_post: gate needed");
   a.gate = (const bf16_t*)gate; a.gs = gate_stride;
   return launch_gemv<PRO_NORMGATE>(a, st);
+}
+
+// The product in front of a parallel layer's sublayers: rows of W below n1 read the shifted h, the others h (and a bias).
+extern "C" int tv_gemv_shift_fwd(const float* x, const void* pending, const void* pending_weight, float* x_out, const void* gain,
+                                 const void* shift, float* state, const int* start, const int* slot, const void* W, const void* bias,
+                                 void* y, int M, int N, int n1, int K, int64_t pending_stride, int64_t state_stride, int64_t ldw,
+                                 int64_t y_stride, float eps, void* stream) {
+  TV_CHECK_ARG(x && gain && shift && state && start && slot && W && y, "gemv_shift: null pointer");
+  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8 && n1 >= 0 && n1 <= N, "gemv_shift: M %d must be 1..%d, N %d >= 1, K %d >= 8", M, GV_MAXM, N, K);
+  TV_CHECK_ARG(!pending || (pending_weight && x_out && x_out != x), "gemv_shift: what waits needs its weight and a stream to be written (not in place)");
+  if (K % 8 || ldw % 8 || pending_stride % 8 || state_stride % 4 || ((uintptr_t)x & 15) || ((uintptr_t)pending & 15) || ((uintptr_t)pending_weight & 15) ||
+      ((uintptr_t)x_out & 15) || ((uintptr_t)shift & 15) || ((uintptr_t)state & 15) || ((uintptr_t)W & 15))
+    TV_UNSUPPORTED("gemv_shift: K and the row strides must be multiples of 8 elements, operands 16-byte aligned");
+  if ((size_t)2 * M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_shift: 2 x M x K = 2 x %d x %d does not fit the 128 KiB of LDS", M, K);
+  if (K > 8 * GV_THREADS * 4) TV_UNSUPPORTED("gemv_shift: rows of <= %d channels", 8 * GV_THREADS * 4);
+  GemvArgs a{};
+  a.W = (const bf16_t*)W; a.bias = (const bf16_t*)bias; a.y = (bf16_t*)y;
+  a.M = M; a.N = N; a.K = K; a.group = K; a.ldw = ldw; a.ys = y_stride; a.eps = eps;
+  a.res = x; a.res_out = x_out; a.delta = (const bf16_t*)pending; a.ds = pending_stride; a.norm_w = pending_weight;
+  a.gain = (const bf16_t*)gain; a.shift = (const bf16_t*)shift; a.state = state; a.sst = state_stride; a.start = start; a.slot = slot;
+  a.N1 = n1;
+  return launch_gemv<PRO_SHIFT>(a, (hipStream_t)stream);
+}
+
+// y = [x | gelu_tanh(z) u] W^T (+ bias); with a residual: residual + y in fp32 (and its bf16 rounding) instead of y.
+extern "C" int tv_gemv_glu_fwd(const void* x, const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W,
+                               const void* bias, const float* residual, float* residual_out, void* h_out, void* y, int M, int N, int k1,
+                               int K, int64_t x_stride, int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream) {
+  TV_CHECK_ARG(W && (x || k1 == 0) && ((z && u) || k1 == K) && (residual ? residual_out != nullptr : y != nullptr), "gemv_glu: null pointer");
+  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8 && k1 >= 0 && k1 <= K && (k1 == K || u_rows > 0),
+               "gemv_glu: M %d must be 1..%d, N %d >= 1, K %d >= 8, %d columns of x", M, GV_MAXM, N, K, k1);
+  if (K % 8 || k1 % 8 || ldw % 8 || x_stride % 8 || z_stride % 8 || u_stride % 8 || ((uintptr_t)x & 15) || ((uintptr_t)z & 15) ||
+      ((uintptr_t)u & 15) || ((uintptr_t)W & 15))
+    TV_UNSUPPORTED("gemv_glu: K, its parts and the row strides must be multiples of 8 elements, operands 16-byte aligned");
+  if ((size_t)M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_glu: M x K = %d x %d does not fit the 128 KiB of LDS f(x) is held in", M, K);
+  GemvArgs a{};
+  a.x = (const bf16_t*)x; a.W = (const bf16_t*)W; a.bias = (const bf16_t*)bias; a.y = (bf16_t*)y;
+  a.M = M; a.N = N; a.K = K; a.group = K; a.xs = x_stride; a.ldw = ldw; a.ys = y_stride;
+  a.res = residual; a.res_out = residual_out; a.h_out = (bf16_t*)h_out;
+  a.K1 = k1; a.z = (const bf16_t*)z; a.u = (const bf16_t*)u; a.u_ids = u_ids; a.zs = z_stride; a.us = u_stride; a.u_rows = u_rows;
+  return launch_gemv<PRO_GLU>(a, (hipStream_t)stream);
 }

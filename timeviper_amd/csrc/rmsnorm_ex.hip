@@ -63,8 +63,6 @@ __device__ __forceinline__ float block_total(float v, float* red) {
   return t;
 }
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
-
 template <typename XT, typename WT, typename YT, bool MOE>
 __global__ __launch_bounds__(RX_THREADS) void rmsnorm_ex_kernel(RxArgs a) {
   __shared__ float red[RX_THREADS / 64];
@@ -161,15 +159,25 @@ __global__ __launch_bounds__(RX_THREADS) void rmsnorm_ex_scalar_kernel(RxArgs a)
   }
 }
 
-// rows of an embedding table times a constant, in fp32 (the residual stream) and in the model's dtype
+// rows of an embedding table times a constant, in fp32 (the residual stream) and in the model's dtype; with a position table
+// its row of the token's place in the sequence is added: place = start[b] + row - cu[b], b = seq[row]
 template <typename T>
 __global__ __launch_bounds__(RX_THREADS) void embed_scaled_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
                                                                   float* __restrict__ x, T* __restrict__ h, int D, int64_t vocab,
-                                                                  float scale) {
+                                                                  float scale, const T* __restrict__ pos, const int* __restrict__ seq,
+                                                                  const int* __restrict__ cu, const int* __restrict__ start,
+                                                                  int64_t max_pos) {
   const int64_t row = blockIdx.x, id = ids[row];
-  const bool ok = id >= 0 && id < vocab;             // (callers check on the host; a bad id reads nothing)
+  const bool ok = id >= 0 && id < vocab;             // (callers check on the host; a bad id or place reads nothing)
+  int64_t at = -1;
+  if (pos) {
+    const int b = seq[row];
+    at = (int64_t)start[b] + row - cu[b];
+    if (at >= max_pos) at = -1;
+  }
   for (int d = threadIdx.x; d < D; d += RX_THREADS) {
-    const float v = ok ? to_f32(table[id * D + d]) * scale : 0.f;
+    float v = ok ? to_f32(table[id * D + d]) * scale : 0.f;
+    if (at >= 0) v += to_f32(pos[at * D + d]);
     x[row * D + d] = v;
     if (h) h[row * D + d] = from_f32<T>(v);
   }
@@ -226,13 +234,17 @@ extern "C" int tv_moe_combine_norm_fwd(const void* expert_out, const int* pos, c
 }
 
 extern "C" int tv_embed_scaled_fwd(const int64_t* ids, const void* table, float* x, void* h, int64_t rows, int D, int64_t vocab,
-                                   float scale, int dtype, void* stream) {
+                                   float scale, const void* pos, const int* seq, const int* cu, const int* start, int64_t max_pos,
+                                   int dtype, void* stream) {
   TV_CHECK_ARG(rows >= 0 && rows < (1ll << 31) && D > 0 && vocab > 0, "embed_scaled: bad sizes");
   if (rows == 0) return TV_OK;
-  TV_CHECK_ARG(ids && table && x, "embed_scaled: null pointer");
+  TV_CHECK_ARG(ids && table && x && (!pos || (seq && cu && start && max_pos > 0)), "embed_scaled: null pointer");
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == TV_F32) embed_scaled_kernel<float><<<dim3((unsigned)rows), RX_THREADS, 0, st>>>(ids, (const float*)table, x, (float*)h, D, vocab, scale);
-  else if (dtype == TV_BF16) embed_scaled_kernel<bf16_t><<<dim3((unsigned)rows), RX_THREADS, 0, st>>>(ids, (const bf16_t*)table, x, (bf16_t*)h, D, vocab, scale);
+  const dim3 grid((unsigned)rows);
+  if (dtype == TV_F32)
+    embed_scaled_kernel<float><<<grid, RX_THREADS, 0, st>>>(ids, (const float*)table, x, (float*)h, D, vocab, scale, (const float*)pos, seq, cu, start, max_pos);
+  else if (dtype == TV_BF16)
+    embed_scaled_kernel<bf16_t><<<grid, RX_THREADS, 0, st>>>(ids, (const bf16_t*)table, x, (bf16_t*)h, D, vocab, scale, (const bf16_t*)pos, seq, cu, start, max_pos);
   else TV_UNSUPPORTED("embed_scaled: dtype %d", dtype);
   TV_LAUNCH_CHECK();
 }

@@ -953,18 +953,111 @@ def moe_combine_norm(expert_out, pos, weights, residual, norm_weight, eps, weigh
     return y, s
 
 
-def embed_scaled(ids, table, scale=1.0):
-    """(fp32 rows, rows in the table's dtype) of `table[ids] * scale`; ids int64 on the GPU."""
-    _gpu(ids, table)
+def embed_scaled(ids, table, scale=1.0, positions=None, plan=None):
+    """(fp32 rows, rows in the table's dtype) of `table[ids] * scale`; ids int64 on the GPU.  `positions` (max, D): the row of the
+    token's place in its sequence is added (plan: the step's `cache.StepPlan`; its places lie within the table)."""
+    _gpu(ids, table, positions)
     flat = ids.reshape(-1).contiguous()
     V, D = table.shape
     if flat.dtype != torch.int64 or not table.is_contiguous():
         raise TimeViperHipError("embed_scaled: int64 ids and a contiguous table")
     x = torch.empty((flat.numel(), D), dtype=torch.float32, device=table.device)
     h = torch.empty((flat.numel(), D), dtype=table.dtype, device=table.device)
-    check(_capi.lib().tv_embed_scaled_fwd(_p(flat), _p(table), _p(x), _p(h), flat.numel(), D, V, float(scale), _dt(table), _stream()),
+    seq = cu = start = None
+    if positions is not None:
+        seq, cu, start = _plan(plan, flat.numel(), "embed_scaled")[:3]
+        if positions.dtype != table.dtype or positions.dim() != 2 or positions.shape[1] != D or not positions.is_contiguous():
+            raise TimeViperHipError("embed_scaled: positions (max, D) of the table's dtype")
+    check(_capi.lib().tv_embed_scaled_fwd(_p(flat), _p(table), _p(x), _p(h), flat.numel(), D, V, float(scale), _p(positions), _p(seq), _p(cu),
+                                          _p(start), 0 if positions is None else positions.shape[0], _dt(table), _stream()),
           "tv_embed_scaled_fwd")
     return x, h
+
+
+# ------------------------------------------------- parallel layers on a 32-bit residual stream
+def _plan(plan, rows, what):
+    """(seq, cu, start, slot) of a step's plan for `rows` packed rows"""
+    B = len(plan.slots)
+    if plan.rows.numel() != rows:
+        raise TimeViperHipError(f"{what}: {rows} rows in a step of {plan.rows.numel()}")
+    for t, n in ((plan.seq, rows), (plan.cu, B + 1), (plan.start, B), (plan.slot, B)):
+        _gpu(t)
+        _i32(t, n, what + " plan")
+    return plan.seq, plan.cu, plan.start, plan.slot
+
+
+def _shift_state(state, plan, D, what):
+    """(slots, 2, D) fp32 blocks, possibly one layer's slice of a wider state: the distance between two blocks"""
+    if (state.dtype != torch.float32 or state.dim() != 3 or state.shape[1:] != (2, D) or state.stride(2) != 1 or state.stride(1) != D
+            or max(plan.slots) >= state.shape[0]):
+        raise TimeViperHipError(f"{what}: a (slots, 2, {D}) fp32 state with dense blocks")
+    return state.stride(0)
+
+
+def norm_shift(x, gain, eps, pending=None, pending_weight=None, shift=None, state=None, plan=None, need_h=True):
+    """x (T, D) fp32 -> (x', h, hs): x' = x + rms(pending) * pending_weight (x itself without `pending`), h = rms(x') * gain (a tensor of one
+    element), hs = h + (h_before - h) * shift with the h of the sequence's previous token (`state` (slots, 2, D) fp32, advanced in
+    place; None without `shift`).  h and hs have the gain's dtype."""
+    _gpu(x, gain, pending, pending_weight, shift, state)
+    T, D = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous() or gain.numel() != 1:
+        raise TimeViperHipError("norm_shift: dense fp32 rows and a gain of one element")
+    xo, ps = None, 0
+    if pending is not None:
+        if pending.shape != x.shape or pending.dtype != gain.dtype or pending.stride(1) != 1 or pending_weight.dtype != gain.dtype:
+            raise TimeViperHipError("norm_shift: pending rows and weight of x's width and the gain's dtype")
+        _vec(pending_weight, D, "norm_shift pending weight")
+        xo, ps = torch.empty_like(x), pending.stride(0)
+    h = torch.empty((T, D), dtype=gain.dtype, device=x.device) if need_h or shift is None else None
+    hs, seq, cu, start, slot, sst = None, None, None, None, None, 0
+    if shift is not None:
+        _vec(shift, D, "norm_shift shift")
+        if shift.dtype != gain.dtype:
+            raise TimeViperHipError("norm_shift: shift of the gain's dtype")
+        hs = torch.empty((T, D), dtype=gain.dtype, device=x.device)
+        seq, cu, start, slot = _plan(plan, T, "norm_shift")
+        sst = _shift_state(state, plan, D, "norm_shift")
+    check(_capi.lib().tv_norm_shift_fwd(
+        _p(x), _p(pending), _p(pending_weight), _p(xo), _p(gain), _p(shift), _p(state if shift is not None else None), _p(seq), _p(cu), _p(start), _p(slot),
+        _p(h), _p(hs), T, D, ps, sst, float(eps), _dt(gain), _stream()), "tv_norm_shift_fwd")
+    return x if xo is None else xo, h, hs
+
+
+def residual_add(x, u):
+    """(x + u in fp32, its rounding to u's dtype); x (T, D) fp32"""
+    _gpu(x, u)
+    if x.dtype != torch.float32 or not x.is_contiguous() or u.shape != x.shape or u.stride(1) != 1:
+        raise TimeViperHipError("residual_add: dense fp32 x and u of its shape")
+    xo, h = torch.empty_like(x), torch.empty(x.shape, dtype=u.dtype, device=x.device)
+    check(_capi.lib().tv_residual_add_fwd(_p(x), _p(u), _p(xo), _p(h), x.shape[0], x.shape[1], u.stride(0), _dt(u), _stream()),
+          "tv_residual_add_fwd")
+    return xo, h
+
+
+ACT_SIGMOID, ACT_GELU_TANH = 0, 1
+
+
+def gated_mul(a, b, act, ids=None, out=None):
+    """f(a) * b over rows, f = sigmoid or the tanh form of gelu; `ids` (int64): row r meets b[ids[r]].  `out`: rows to write to."""
+    _gpu(a, b, ids, out)
+    T, n = a.shape
+    o = torch.empty((T, n), dtype=a.dtype, device=a.device) if out is None else out
+    if (b.dtype != a.dtype or b.dim() != 2 or b.shape[1] != n or o.shape != a.shape or o.dtype != a.dtype or any(t.stride(1) != 1 for t in (a, b, o))
+            or (ids is None and b.shape[0] != T) or (ids is not None and (ids.dtype != torch.int64 or ids.numel() != T or not ids.is_contiguous()))):
+        raise TimeViperHipError(f"gated_mul: a {tuple(a.shape)} against b {tuple(b.shape)}")
+    check(_capi.lib().tv_gated_mul_fwd(_p(a), _p(b), _p(ids), _p(o), T, n, a.stride(0), b.stride(0), o.stride(0), b.shape[0], int(act), _dt(a),
+                                       _stream()), "tv_gated_mul_fwd")
+    return o
+
+
+def scatter_rows(src, rows, dst):
+    """dst[rows] = src (rows int32 on the GPU, within dst)"""
+    _gpu(src, rows, dst)
+    _i32(rows, src.shape[0], "scatter_rows rows")
+    if src.dtype != dst.dtype or src.shape[1] != dst.shape[1] or src.stride(1) != 1 or dst.stride(1) != 1:
+        raise TimeViperHipError("scatter_rows: rows of one width and dtype")
+    check(_capi.lib().tv_scatter_rows(_p(src), _p(rows), _p(dst), src.shape[0], src.shape[1], src.stride(0), dst.stride(0), _dt(src), _stream()),
+          "tv_scatter_rows")
 
 
 # ------------------------------------------------- linear attention with a constant decay per head
@@ -996,10 +1089,15 @@ def lightning_attention(q, k, v, decay, state, cu_seqlens, slot, nheads, max_len
 
 
 # ------------------------------------------------- attention without shape limits, latent attention
-def attention_generic(q, k, v, cu_seqlens, scale, causal=True, sink=None, start=None, slot=None):
+NO_WINDOW = 2 ** 31 - 1
+
+
+def attention_generic(q, k, v, cu_seqlens, scale, causal=True, sink=None, start=None, slot=None, window=NO_WINDOW, keep_first=0, gate=None,
+                      out=None):
     """q (T, Hq, dk) packed rows of B sequences (cu_seqlens (B + 1) int32); k (blocks, Lk, Hkv, dk), v (blocks, Lk, Hkv, dv): sequence b
-    reads block slot[b] (default b).  Row i of a sequence sees keys [0, start[b] + i] when causal.  Returns (T, Hq, dv)."""
-    _gpu(q, k, v, cu_seqlens, sink, start, slot)
+    reads block slot[b] (default b).  Row i of a sequence sees keys [0, start[b] + i] when causal — with a window, the last `window` of
+    them and the first `keep_first`.  gate (T, Hq, dv): the result times sigmoid(gate).  Returns (T, Hq, dv)."""
+    _gpu(q, k, v, cu_seqlens, sink, start, slot, gate, out)
     T, Hq, dk = q.shape
     B = cu_seqlens.numel() - 1
     Hkv, dv = k.shape[2], v.shape[3]
@@ -1011,12 +1109,90 @@ def attention_generic(q, k, v, cu_seqlens, scale, causal=True, sink=None, start=
         if sink.dtype != torch.float32:
             raise TimeViperHipError("attention_generic: fp32 sinks")
         _vec(sink, Hq, "attention_generic sink")
-    o = torch.empty((T, Hq, dv), dtype=q.dtype, device=q.device)
+    o = torch.empty((T, Hq, dv), dtype=q.dtype, device=q.device) if out is None else out
+    for t in (o, gate):
+        if t is not None and (t.shape != (T, Hq, dv) or t.dtype != q.dtype or t.stride(2) != 1):
+            raise TimeViperHipError("attention_generic: gate and out (T, Hq, dv) of q's dtype with dense last dims")
     check(_capi.lib().tv_attn_generic_fwd(
         _p(q), _p(k), _p(v), _p(sink), _p(o), _p(cu_seqlens), _p(start), _p(slot), B, T, Hq, Hkv, dk, dv, q.stride(0), q.stride(1),
         k.stride(0), k.stride(1), k.stride(2), v.stride(0), v.stride(1), v.stride(2), o.stride(0), o.stride(1), float(scale),
-        int(bool(causal)), _dt(q), _stream()), "tv_attn_generic_fwd")
+        int(bool(causal)), int(window), int(keep_first), _p(gate), 0 if gate is None else gate.stride(0),
+        0 if gate is None else gate.stride(1), _dt(q), _stream()), "tv_attn_generic_fwd")
     return o
+
+
+def _cache_views(cache, kv_heads, dim, vdim):
+    """keys (slots, capacity, kv_heads, dim) and values (slots, capacity, kv_heads, vdim) of rows that hold both side by side"""
+    slots, cap, W = cache.shape
+    if W != kv_heads * (dim + vdim) or not cache.is_contiguous():
+        raise TimeViperHipError(f"cache rows of {W} elements for {kv_heads} x ({dim} + {vdim})")
+    k, v = cache.split([kv_heads * dim, kv_heads * vdim], dim=2)
+    return k.unflatten(2, (kv_heads, dim)), v.unflatten(2, (kv_heads, vdim))
+
+
+def attention_window(q, cache, plan, kv_heads, scale, window=NO_WINDOW, keep_first=0, gate=None, out=None):
+    """Causal attention of a step's packed rows against a slot cache that already holds the step's own keys and values: q (T, H, dk), cache
+    (slots, capacity, kv_heads * (dk + dv)), a row = all keys, then all values; the query at position p sees keys (p - window, p]
+    and the first `keep_first` of its sequence.  gate (T, H, dv): the result times sigmoid(gate).  out (T, H, dv).  plan: the step's
+    `cache.StepPlan`."""
+    T, H, dk = q.shape
+    dv = cache.shape[2] // kv_heads - dk
+    k, v = _cache_views(cache, kv_heads, dk, dv)
+    _, cu, start, slot = _plan(plan, T, "attention_window")
+    if max(plan.slots) >= cache.shape[0] or max(a + n for a, n in zip(plan.starts, plan.counts)) > cache.shape[1]:
+        raise TimeViperHipError("attention_window: the cache does not hold the step's tokens")
+    o = torch.empty((T, H, dv), dtype=q.dtype, device=q.device) if out is None else out
+    rows8 = lambda t: t is None or (all(s % 4 == 0 for s in t.stride()[:2]) and t.data_ptr() % 8 == 0 and t.stride(2) == 1)
+    if not (q.dtype == torch.bfloat16 and cache.dtype == q.dtype and _flash_rows(q) and _flash_rows(k[0]) and _flash_rows(v[0]) and rows8(gate)
+            and rows8(o) and scale > 0):
+        return attention_generic(q, k, v, cu, scale, start=start, slot=slot, window=window, keep_first=keep_first, gate=gate, out=o)
+    _gpu(q, cache, gate, o)
+    if H % kv_heads or any(t is not None and (t.shape != (T, H, dv) or t.dtype != q.dtype) for t in (gate, o)):
+        raise TimeViperHipError("attention_window: gate and out (T, H, dv) of q's dtype")
+    lib, at = _capi.lib(), 0
+    for s, n, a in zip(plan.slots, plan.counts, plan.starts):
+        sl = slice(at, at + n)
+        gb = None if gate is None else gate[sl]
+        check(lib.tv_flash_attn_window_fwd(
+            _p(q[sl]), _p(k[s]), _p(v[s]), _p(o[sl]), _p(gb), int(window), int(keep_first), dv, n, a + n, H, kv_heads, dk, q.stride(0), q.stride(1),
+            k.stride(1), k.stride(2), v.stride(1), v.stride(2), o.stride(0), o.stride(1), 0 if gate is None else gate.stride(0),
+            0 if gate is None else gate.stride(1), float(scale), _dt(q), _stream()), "tv_flash_attn_window_fwd")
+        at += n
+    return o
+
+
+def attention_window_decode(q, cache, plan, kv_heads, scale, window=NO_WINDOW, keep_first=0, gate=None, fresh=None, out=None):
+    """`attention_window` for a step of single tokens: q (B, H, dk), gate (B, H, dv).  fresh (B, kv_heads * (dk + dv)): the step's own cache
+    rows, which are written here (without it they are in the cache already).  Key counts are read on the device.  Returns (B, H, dv)
+    (`out`: where to)."""
+    B, H, dk = q.shape
+    dv = cache.shape[2] // kv_heads - dk
+    k, v = _cache_views(cache, kv_heads, dk, dv)
+    _, cu, start, slot = _plan(plan, B, "attention_window_decode")
+    if not plan.decode or max(plan.slots) >= cache.shape[0] or H % kv_heads:
+        raise TimeViperHipError("attention_window_decode: one token per sequence, each with a slot of the cache")
+    _gpu(q, cache, gate, fresh, out, plan.keys)
+    _i32(plan.keys, B, "attention_window_decode keys")
+    if fresh is not None and (fresh.shape != (B, cache.shape[2]) or fresh.dtype != cache.dtype or fresh.stride(1) != 1):
+        raise TimeViperHipError("attention_window_decode: new rows of the cache's width and dtype")
+    dense = lambda t: t is None or (t.stride(2) == 1 and t.stride(1) == t.shape[2])
+    ok16 = lambda t: t is None or (t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0)
+    if (q.dtype == torch.bfloat16 and cache.dtype == q.dtype and dk % 8 == 0 and dv % 8 == 0 and max(dk, dv) <= 256 and dense(q) and dense(gate)
+            and dense(out) and ok16(q) and ok16(fresh) and ok16(cache)):
+        if any(t is not None and (t.shape != (B, H, dv) or t.dtype != q.dtype) for t in (gate, out)):
+            raise TimeViperHipError("attention_window_decode: gate and out (B, H, dv) of q's dtype")
+        o = torch.empty((B, H, dv), dtype=q.dtype, device=q.device) if out is None else out
+        lib, cap = _capi.lib(), cache.shape[1]
+        nbytes = int(lib.tv_attn_window_decode_workspace_bytes(B, H, kv_heads, dv, cap, int(window), int(keep_first)))
+        ws = torch.empty(nbytes, dtype=torch.uint8, device=q.device) if nbytes else None
+        check(lib.tv_attn_window_decode_fwd(
+            _p(q), _p(cache), _p(fresh), _p(gate), _p(o), _p(plan.keys), _p(slot), B, H, kv_heads, dk, dv, cap, int(window), int(keep_first),
+            q.stride(0), 0 if fresh is None else fresh.stride(0), 0 if gate is None else gate.stride(0), o.stride(0), float(scale), _p(ws), nbytes,
+            _stream()), "tv_attn_window_decode_fwd")
+        return o
+    if fresh is not None:
+        scatter_rows(fresh, plan.rows, cache.view(-1, cache.shape[2]))
+    return attention_generic(q, k, v, cu, scale, start=start, slot=slot, window=window, keep_first=keep_first, gate=gate, out=out)
 
 
 def _flash_rows(t: torch.Tensor) -> bool:
@@ -1158,6 +1334,74 @@ def gemv_post(x, weight, prologue=GEMV_NONE, residual=None, norm_weight=None, ep
         _p(norm_weight), 0 if norm_weight is None else _dt(norm_weight), float(weight_offset), float(mult), float(eps), _p(gate),
         0 if gate is None else gate.stride(0), _stream()), "tv_gemv_post_fwd")
     return (y, xs, hs) if prologue == GEMV_POSTNORM else y
+
+
+def gemv_shift_takes(rows: int, width: int, dtype) -> bool:
+    """Shapes of tv_gemv_shift_fwd: 1..4 bf16 rows of up to 8 192 elements, twice in LDS."""
+    return dtype == torch.bfloat16 and 1 <= rows <= 4 and width % 8 == 0 and width <= 8192 and rows * width * 4 <= 128 * 1024
+
+
+def gemv_shift(x, gain, eps, shift, state, plan, weight, n1, bias=None, pending=None, pending_weight=None):
+    """`norm_shift` and the product behind it for single tokens (1..4): (x', y) with y = [hs @ weight[:n1].T | h @ weight[n1:].T + bias], bf16."""
+    _gpu(x, gain, shift, state, weight, bias, pending, pending_weight)
+    M, D = x.shape
+    N = weight.shape[0]
+    bf = torch.bfloat16
+    if (x.dtype != torch.float32 or not x.is_contiguous() or weight.dtype != bf or weight.shape[1] != D or weight.stride(1) != 1 or gain.dtype != bf
+            or gain.numel() != 1 or shift.dtype != bf or not plan.decode or (bias is not None and bias.dtype != bf)):
+        raise TimeViperHipError(f"gemv_shift: dense fp32 rows {tuple(x.shape)} against a bf16 weight {tuple(weight.shape)}")
+    _vec(shift, D, "gemv_shift shift")
+    if bias is not None:
+        _vec(bias, N - n1, "gemv_shift bias")
+    xo, ps = None, 0
+    if pending is not None:
+        if pending.shape != x.shape or pending.dtype != bf or pending.stride(1) != 1 or pending_weight.dtype != bf:
+            raise TimeViperHipError("gemv_shift: pending rows and weight in bf16, of x's width")
+        _vec(pending_weight, D, "gemv_shift pending weight")
+        xo, ps = torch.empty_like(x), pending.stride(0)
+    _, _, start, slot = _plan(plan, M, "gemv_shift")
+    sst = _shift_state(state, plan, D, "gemv_shift")
+    y = torch.empty((M, N), dtype=bf, device=x.device)
+    check(_capi.lib().tv_gemv_shift_fwd(
+        _p(x), _p(pending), _p(pending_weight), _p(xo), _p(gain), _p(shift), _p(state), _p(start), _p(slot), _p(weight), _p(bias), _p(y), M, N, int(n1),
+        D, ps, sst, weight.stride(0), N, float(eps), _stream()), "tv_gemv_shift_fwd")
+    return x if xo is None else xo, y
+
+
+def gemv_glu_takes(rows: int, k1: int, k2: int, dtype) -> bool:
+    """Shapes of tv_gemv_glu_fwd."""
+    return dtype == torch.bfloat16 and 1 <= rows <= 4 and k1 % 8 == 0 and k2 % 8 == 0 and rows * (k1 + k2) * 2 <= 128 * 1024
+
+
+def gemv_glu(x, z, u, weight, bias=None, residual=None, ids=None):
+    """y = [x | gelu_tanh(z) * u] @ weight.T + bias for 1..4 bf16 rows; x or (z, u) may be None; `ids` (int64): row m meets u[ids[m]].  With
+    `residual` (fp32): (residual + y in fp32, its bf16 rounding), else y in bf16."""
+    _gpu(x, z, u, weight, bias, residual, ids)
+    bf = torch.bfloat16
+    M = (x if x is not None else z).shape[0]
+    N, Kd = weight.shape
+    k1 = 0 if x is None else x.shape[1]
+    if (k1 + (0 if z is None else z.shape[1]) != Kd or weight.dtype != bf or weight.stride(1) != 1 or (z is None) != (u is None)
+            or any(t is not None and (t.dtype != bf or t.stride(1) != 1) for t in (x, z, u)) or any(t is not None and t.shape[0] != M for t in (x, z))
+            or (u is not None and (u.shape[1] != z.shape[1] or (ids is None and u.shape[0] != M)))
+            or (ids is not None and (ids.dtype != torch.int64 or ids.numel() != M or not ids.is_contiguous()))):
+        raise TimeViperHipError(f"gemv_glu: bf16 rows that make up the {Kd} columns of the weight")
+    if bias is not None:
+        _vec(bias, N, "gemv_glu bias")
+        if bias.dtype != bf:
+            raise TimeViperHipError("gemv_glu: bf16 bias")
+    y = xo = ho = None
+    if residual is not None:
+        if residual.dtype != torch.float32 or residual.shape != (M, N) or not residual.is_contiguous():
+            raise TimeViperHipError("gemv_glu: a dense fp32 residual (M, N)")
+        xo, ho = torch.empty_like(residual), torch.empty((M, N), dtype=bf, device=residual.device)
+    else:
+        y = torch.empty((M, N), dtype=bf, device=weight.device)
+    st = lambda t: 0 if t is None else t.stride(0)
+    check(_capi.lib().tv_gemv_glu_fwd(
+        _p(x), _p(z), _p(u), _p(ids), 0 if u is None else u.shape[0], _p(weight), _p(bias), _p(residual), _p(xo), _p(ho), _p(y), M, N, k1, Kd, st(x),
+        st(z), st(u), weight.stride(0), N, _stream()), "tv_gemv_glu_fwd")
+    return y if residual is None else (xo, ho)
 
 
 # ------------------------------------------------- mixture of experts

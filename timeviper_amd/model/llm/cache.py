@@ -57,6 +57,7 @@ class StepPlan:
     start: torch.Tensor            # (B) int32
     slot: torch.Tensor             # (B) int32
     rows: torch.Tensor             # (T) int32: cache row of every new token in a (slots * capacity, width) view
+    seq: torch.Tensor              # (T) int32: the sequence (index into slots) of every new token
     keys: Optional[torch.Tensor]   # (B) int32, start + 1: keys in use after a single-token step
     moving: Optional[torch.Tensor] # (3, B) int32 behind start, rows and keys of a single-token step: what a step adds 1 to
     decode: bool                   # one token per sequence
@@ -77,10 +78,13 @@ class StepPlan:
 
 class SlotStateCache(StaticDecode):
     """`layers[i]`: ("tokens", width) — a (slots, capacity, width) buffer of the model's dtype — or ("state", shape) — a
-    (slots, *shape) fp32 block, zero when a sequence starts.  Buffers grow geometrically unless static decode fixed them."""
+    (slots, *shape) fp32 block, zero when a sequence starts.  (Entries need not be the model's layers: several layers may read one
+    entry, or none.)  Buffers grow geometrically unless static decode fixed them.  `limit`: the most tokens a sequence may have
+    (a learned position table); a step beyond it is refused."""
 
     def __init__(self, layers: Sequence[Tuple[str, object]], slots: int = 1, dtype=torch.bfloat16, device=None,
-                 capacity: int = 0, reserve: int = 256):
+                 capacity: int = 0, reserve: int = 256, limit: Optional[int] = None):
+        self.limit = limit
         self.layers, self.dtype, self.device = list(layers), dtype, device
         self.reserve = int(reserve)
         self.capacity, self.num_slots = 0, 0
@@ -163,23 +167,28 @@ class SlotStateCache(StaticDecode):
         starts = tuple(self._len[s] for s in slots)
         single = all(c == 1 for c in counts)
         dp = self._decode_plan
-        if single and dp is not None and dp.slots == slots and dp.starts == starts and max(starts) < self.capacity:
+        if single and dp is not None and dp.slots == slots and dp.starts == starts and max(starts) < min(self.capacity, self.limit or self.capacity):
             return dp
         if self.static_decode:
             raise RuntimeError("static decode takes one token of the same sequences every step")
         need = max(a + c for a, c in zip(starts, counts))
+        if self.limit is not None and need > self.limit:
+            raise ValueError(f"a sequence of {need} tokens: this model takes at most {self.limit}")
         if need > self.capacity:
-            self._resize(self.num_slots, need + max(self.reserve, need // 8))
+            room = need + max(self.reserve, need // 8)
+            self._resize(self.num_slots, room if self.limit is None else min(room, self.limit))
         i32 = lambda v: torch.tensor(v, dtype=torch.int32).to(self.device)
-        cu, rows = [0], []
-        for s, a, c in zip(slots, starts, counts):
+        cu, rows, seq = [0], [], []
+        for b, (s, a, c) in enumerate(zip(slots, starts, counts)):
             cu.append(cu[-1] + c)
             rows.append(torch.arange(s * self.capacity + a, s * self.capacity + a + c, dtype=torch.int32))
+            seq.append(torch.full((c,), b, dtype=torch.int32))
+        seq = torch.cat(seq).to(self.device)
         if single:
             mv = i32([list(starts), [s * self.capacity + a for s, a in zip(slots, starts)], [a + 1 for a in starts]])
-            p = StepPlan(slots, counts, starts, i32(cu), mv[0], i32(slots), mv[1], mv[2], mv, True)
+            p = StepPlan(slots, counts, starts, i32(cu), mv[0], i32(slots), mv[1], seq, mv[2], mv, True)
         else:
-            p = StepPlan(slots, counts, starts, i32(cu), i32(starts), i32(slots), torch.cat(rows).to(self.device), None, None, False)
+            p = StepPlan(slots, counts, starts, i32(cu), i32(starts), i32(slots), torch.cat(rows).to(self.device), seq, None, None, False)
         if single:
             self._decode_plan = p
         return p
@@ -204,6 +213,8 @@ class SlotStateCache(StaticDecode):
             raise RuntimeError("static decode starts behind a prefill (every sequence holding its tokens)")
         self.end_static_decode()
         need = max(self._len[s] for s in slots) + int(max_new_tokens)
+        if self.limit is not None:
+            need = min(need, self.limit)
         if need > self.capacity:
             self._resize(self.num_slots, need)
         self._decode_plan = None
@@ -214,7 +225,7 @@ class SlotStateCache(StaticDecode):
         self.static_decode = False
 
     def static_room(self) -> int:
-        return self.capacity - max(self._len[s] for s in self.default_slots)
+        return min(self.capacity, self.limit or self.capacity) - max(self._len[s] for s in self.default_slots)
 
     def advance_static_device(self):
         self._advance_device(self._decode_plan)

@@ -1,6 +1,6 @@
 """Language models from a folder: config.json + model.safetensors.
 
-The model class is chosen by config.json: "architecture" (Fasovik) or "model_type" (nano, qwen2).  A model names its
+The model class is chosen by config.json: "architecture" (Fasovik, Fogorax) or "model_type" (nano, qwen2).  A model names its
 checkpoint tensors in `checkpoint_tensors()` — views into its (possibly stacked) parameters — or, without that method, by
 its parameter names.  Loading is strict: every tensor of the file has one place, every place is filled, shapes agree."""
 from __future__ import annotations

@@ -24,11 +24,12 @@ class TextEngine:
         self.llm, self.device = llm, llm.device
         self.ragged = bool(getattr(llm, "supports_ragged", False))
         self._live: Dict[Hashable, object] = {}             # request -> slot, or (cache, tokens seen) of its own
-        self.cache = None
+        self.cache, self.limit = None, None                 # limit: the most tokens of one request
         if self.ragged:
             self.cache = llm.new_cache(0)
+            self.limit = self.cache.limit
             # (max_tokens bounds the longest request as well; buffers grow when a step needs more)
-            self.cache._resize(slots, min(int(max_tokens or 0), 4096))
+            self.cache._resize(slots, min(int(max_tokens or 0), 4096, self.limit or 4096))
 
     def _check(self, tokens):
         if not len(tokens) or min(tokens) < 0 or max(tokens) >= self.llm.config.vocab_size:
@@ -39,8 +40,10 @@ class TextEngine:
         """fp32 logits (wanted places, vocab), in the order of the entries and of their places."""
         if not entries:
             return torch.empty((0, self.llm.config.vocab_size), device=self.device)
-        for _, tokens, want in entries:
+        for rid, tokens, want in entries:
             self._check(tokens)
+            if self.limit is not None and (self.cache.length(self._live[rid]) if rid in self._live else 0) + len(tokens) > self.limit:
+                raise ValueError(f"request {rid!r}: this model takes at most {self.limit} tokens a request")
             if any(not 0 <= w < len(tokens) for w in want):
                 raise ValueError("a wanted place lies outside the step's tokens")
         return self._step_packed(entries) if self.ragged else self._step_each(entries)
@@ -84,9 +87,12 @@ class TextEngine:
         out: List[List[int]] = [[] for _ in prompts]
         running: List[int] = []
 
+        def most(i):                                         # new tokens request i may get: one behind its last place is never fed back
+            return max_new_tokens if self.limit is None else min(max_new_tokens, self.limit - len(prompts[i]) + 1)
+
         def take(i, token):                                  # True: request i goes on
             out[i].append(token)
-            return token not in eos and len(out[i]) < max_new_tokens
+            return token not in eos and len(out[i]) < most(i)
 
         if max_new_tokens < 1:
             return out
@@ -102,7 +108,7 @@ class TextEngine:
                     else:
                         self.end(("gen", i))
                 continue
-            left = max(max_new_tokens - len(out[i]) for i in running)
+            left = max(most(i) - len(out[i]) for i in running)
             stepper = self._stepper(running, left) if not waiting else None
             if stepper is not None:                          # nobody joins any more: finished requests ride along
                 self._replay(stepper, running, take, out)
@@ -124,6 +130,8 @@ class TextEngine:
         if (not self.ragged or left < 8 or self.device.type != "cuda" or os.environ.get("TV_DECODE_GRAPH", "1") == "0"
                 or not self.llm.graph_decode_supported(self.cache)):
             return None
+        if self.limit is not None and max(self.cache.length(self._live[("gen", i)]) for i in running) + left > self.limit:
+            return None                                      # (finished requests ride along: not past the last place)
         cache, vocab = self.cache, self.llm.config.vocab_size
         cache.default_slots = tuple(self._live[("gen", i)] for i in running)
         cache.begin_static_decode(left)

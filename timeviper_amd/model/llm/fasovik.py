@@ -7,23 +7,20 @@ residual stream; only what a sublayer returns is normalised:
 Layers may share one set of parameters ("weights_of"); their caches and states stay separate.  Embedding rows are scaled on
 the way in; the logits use the table as it is.
 
-Steps are PACKED: the new tokens of all sequences of a step are consecutive rows, without padding; `cache.StepPlan` says
-which sequence and which cache rows they belong to.  The usual (batch, tokens) calls of the framework's other models are
-accepted as well (`forward`)."""
+Steps are packed (packed.py)."""
 from __future__ import annotations
 
 import os
-from typing import Any, List, Optional, Sequence
+from typing import List, Optional, Sequence
 
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
 from ... import kernels as K
 from .cache import SlotStateCache
 from .mixers import DecodeStream, LatentAttention, LightningAttention, _weight
 from .moe import MixtureOfExperts
-from .nano import CausalLMOutputWithPast
+from .packed import PackedCausalLM, vocabulary_logits
 
 NORM_OFFSET = 1.0            # the norms' weights are stored around zero
 
@@ -165,9 +162,7 @@ class FasovikModel(nn.Module):
         return x, h
 
 
-class FasovikForCausalLM(nn.Module):
-    supports_ragged = True       # sequences of different lengths share a step (engine.py)
-
+class FasovikForCausalLM(PackedCausalLM):
     def __init__(self, config: FasovikConfig):
         super().__init__()
         if config.use_pdrop or config.merge_module != "no_merge":
@@ -214,14 +209,7 @@ class FasovikForCausalLM(nn.Module):
         cache.alloc_batch(batch_size)
         return cache
 
-    def graph_decode_supported(self, cache) -> bool:
-        """A decode step has fixed launch parameters: positions and key counts are read on the device."""
-        return isinstance(cache, SlotStateCache)
-
-    # ---- one packed step
-    def step(self, ids, cache: SlotStateCache, plan, logits_at=None, embeds=None, trace: Optional[list] = None):
-        """New tokens of the sequences of `plan` (ids (T) int64, or embeds (T, width)): logits fp32 at the rows `logits_at`
-        (int64 tensor; None: every row)."""
+    def hidden(self, ids, cache, plan, logits_at=None, embeds=None, trace=None):
         if embeds is None:
             x, h = self.backbone.embed.rows(ids)
         else:
@@ -229,53 +217,7 @@ class FasovikForCausalLM(nn.Module):
         if trace is not None:
             trace.append(x)
         x, h = self.backbone(x, h, cache, plan, trace)
-        cache.commit(plan)
-        if logits_at is not None:
-            x = x.index_select(0, logits_at)
-        return self.logits(x)
+        return x if logits_at is None else x.index_select(0, logits_at)
 
     def logits(self, x):
-        h = K.rms_norm_ex(x, self.backbone.final_norm, self.config.norm_eps, NORM_OFFSET)
-        if K.gemv_post_takes(h.shape[0], h.shape[1], h.dtype):
-            return K.gemv_post(h, self.backbone.embed.weight, out_dtype=torch.float32)
-        return F.linear(h, self.backbone.embed.weight).float()
-
-    # ---- the (batch, tokens) call of the framework's other models
-    def forward(self, input_ids=None, inputs_embeds=None, attention_mask=None, position_ids=None, past_key_values=None,
-                labels=None, use_cache=None, cache_position=None, logits_to_keep=None, output_hidden_states=None,
-                train_pdrop_args: Any = None, **kwargs):
-        """input_ids (B, L) or inputs_embeds (B, L, width): the next L tokens of every sequence of the cache (a new one without
-        `past_key_values`).  attention_mask (B, L) with zeros marks padding rows on either side: they are left out, and their
-        logits are zero.  logits_to_keep: the last n positions (default `num_logits_to_keep`; 0: all)."""
-        if (input_ids is None) == (inputs_embeds is None):
-            raise ValueError("You must specify exactly one of input_ids or inputs_embeds")
-        if labels is not None:
-            raise NotImplementedError("loss computation is a training feature")
-        src = input_ids if inputs_embeds is None else inputs_embeds
-        B, L = src.shape[:2]
-        cache = past_key_values if past_key_values is not None else self.new_cache(B)
-        if len(cache.default_slots) != B:
-            raise ValueError(f"the cache holds {len(cache.default_slots)} sequences, the call {B}")
-        keep = None
-        flat = src.reshape(B * L, *src.shape[2:])
-        counts = [L] * B
-        if attention_mask is not None and not bool(attention_mask.all()):
-            m = attention_mask.bool()
-            counts = [int(c) for c in m.sum(1)]
-            keep = m.reshape(-1).nonzero().flatten()
-            flat = flat.index_select(0, keep)
-        plan = cache.plan(cache.default_slots, counts)
-        trace = [] if output_hidden_states else None
-        n = self.config.num_logits_to_keep if logits_to_keep is None else int(logits_to_keep)
-        kw = dict(ids=flat.contiguous()) if inputs_embeds is None else dict(ids=None, embeds=flat)
-        if keep is None:
-            at = None
-            if 0 < n < L:
-                at = (torch.arange(B, device=src.device)[:, None] * L + torch.arange(L - n, L, device=src.device)).flatten()
-            logits = self.step(cache=cache, plan=plan, logits_at=at, trace=trace, **kw).view(B, -1, self.vocab_size)
-        else:
-            packed = self.step(cache=cache, plan=plan, trace=trace, **kw)
-            logits = packed.new_zeros((B * L, self.vocab_size)).index_copy_(0, keep, packed).view(B, L, -1)
-            logits = logits[:, -n:] if n > 0 else logits
-        return CausalLMOutputWithPast(loss=None, logits=logits, past_key_values=cache if use_cache is not False else None,
-                                      hidden_states=None if trace is None else tuple(trace))
+        return vocabulary_logits(K.rms_norm_ex(x, self.backbone.final_norm, self.config.norm_eps, NORM_OFFSET), self.backbone.embed.weight)

@@ -11,6 +11,7 @@ import torch
 import torch.nn as nn
 
 from .fasovik import FasovikConfig, FasovikForCausalLM
+from .fogorax import FogoraxConfig, FogoraxForCausalLM
 from .nano import NemotronHConfig, NemotronHForCausalLM
 from .qwen2 import Qwen2Config, Qwen2ForCausalLM
 
@@ -19,6 +20,7 @@ LLM_FAMILIES = {
     "nano": (NemotronHConfig, NemotronHForCausalLM),
     "qwen2": (Qwen2Config, Qwen2ForCausalLM),
     "fasovik": (FasovikConfig, FasovikForCausalLM),
+    "fogorax": (FogoraxConfig, FogoraxForCausalLM),
 }
 
 MODEL_REGISTRY = {
@@ -34,7 +36,8 @@ QWEN2_REGISTRY = {
     "qwen2.5-7b-instruct": "Qwen/Qwen2.5-7B-Instruct", "qwen2.5-7b-base": "Qwen/Qwen2.5-7B-Base",
     "qwen2.5-3b-instruct": "Qwen/Qwen2.5-3B-Instruct", "qwen2.5-3b-base": "Qwen/Qwen2.5-3B-Base",
 }
-FASOVIK_REGISTRY = {"fasovik": "Fasovik"}      # sizes come with a configuration (`config=`, or a checkpoint folder)
+# layer-list designs: sizes come with a configuration (`config=`, or a checkpoint folder)
+LAYER_LIST_REGISTRY = {"fasovik": "Fasovik", "fogorax": "Fogorax"}
 _QWEN2_7B = ("qwen2-7b", "qwen2-7b-instruct", "qwen2.5-7b-instruct", "qwen2.5-7b-base")
 DEFAULT_TOKEN = "<image>"
 
@@ -44,8 +47,8 @@ def llm_family_of(llm_backbone_id: str) -> str:
         return "nano"
     if llm_backbone_id in QWEN2_REGISTRY:
         return "qwen2"
-    if llm_backbone_id in FASOVIK_REGISTRY:
-        return "fasovik"
+    if llm_backbone_id in LAYER_LIST_REGISTRY:
+        return llm_backbone_id
     raise ValueError(f"LLM backbone `{llm_backbone_id}` is not supported!")
 
 

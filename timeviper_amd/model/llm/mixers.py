@@ -1,5 +1,5 @@
-"""Token mixers of the layer-list models (fasovik.py): linear attention with a constant decay per head, and latent
-attention with sinks.  A mixer reads the packed rows of a step (`cache.StepPlan`), keeps its state in a `SlotStateCache`
+"""Token mixers of the layer-list models (fasovik.py, fogorax.py): linear attention with a constant decay per head, latent
+attention with sinks, and attention in a sliding window with kept first tokens.  A mixer reads the packed rows of a step (`cache.StepPlan`), keeps its state in a `SlotStateCache`
 layer and returns one row per token; every constant is a constructor argument.
 
 A mixer offers
@@ -8,10 +8,12 @@ A mixer offers
     decode(stream, cache, layer, plan)   the same for a few single tokens, on the fused matrix-vector kernels (`DecodeStream`)
     checkpoint_tensors()              (name in a checkpoint, view of a parameter) pairs: projections that share their input
                                       are one stacked parameter
-"""
+
+A mixer of a layer whose sublayers run in parallel (`WindowAttention`, parallel.py) has no parameters of its own: its
+projections are rows and columns of the layer's stacked matrices."""
 from __future__ import annotations
 
-from typing import Sequence
+from typing import Optional, Sequence
 
 import torch
 import torch.nn as nn
@@ -21,7 +23,7 @@ from ... import kernels as K
 
 
 def _weight(*shape) -> nn.Parameter:
-    return nn.Parameter(torch.empty(*shape))
+    return nn.Parameter(torch.empty(shape))
 
 
 class DecodeStream:
@@ -160,3 +162,46 @@ class LatentAttention(nn.Module):
         k, v = kv.split([self.nk, self.nv], dim=1)
         k, v = k.unflatten(1, (self.heads, self.dim)), v.unflatten(1, (self.heads, self.vdim))
         return K.attention_sink(q, k, v, cu_q, cu_k, start, counts, starts, self.scale, self.sink32())
+
+
+class WindowAttention:
+    """Softmax attention without positions; query heads share key / value heads in groups.  The query at position p sees the last
+    `window` keys up to its own and the first `keep_first` of the sequence (window None: all); the concatenated heads are
+    multiplied by a sigmoid gate.  The cache holds keys and values side by side; a mixer without `own_kv` has no key and value
+    projections and reads another layer's rows, which the step has already written.
+
+    Its projections q | k | v | gate are `in_rows` rows of the layer's input matrix, the output projection `out_cols` columns of
+    the output matrix."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, window: Optional[int] = None, keep_first: int = 0,
+                 own_kv: bool = True):
+        if heads % kv_heads or (window is not None and window < 1) or keep_first < 0:
+            raise ValueError(f"window attention: {heads} heads on {kv_heads} key / value heads, window {window}, {keep_first} kept")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.scale, self.own_kv = heads, kv_heads, dim, vdim, float(scale), own_kv
+        self.window, self.keep_first = K.NO_WINDOW if window is None else int(window), int(keep_first)
+        self.nq, self.nv = heads * dim, heads * vdim
+        self.cache_width = kv_heads * (dim + vdim)
+        self.parts = [self.nq, self.cache_width if own_kv else 0, self.nv]
+        self.in_rows, self.out_cols = sum(self.parts), self.nv
+
+    def checkpoint_tensors(self, inp, out):
+        q, kv, g = inp.split(self.parts)
+        got = [("q", q), ("g", g), ("o", out)]
+        if self.own_kv:
+            k, v = kv.split([self.kv_heads * self.dim, self.kv_heads * self.vdim])
+            got += [("k", k), ("v", v)]
+        return got
+
+    def attend(self, p, rows, plan, out=None):
+        """p (T, in_rows): the projections; rows: the cache entry of the layer's keys and values -> the gated heads (T, out_cols)"""
+        q, kv, g = p.split(self.parts, dim=1)
+        q, g = q.unflatten(1, (self.heads, self.dim)), g.unflatten(1, (self.heads, self.vdim))
+        o = None if out is None else out.unflatten(1, (self.heads, self.vdim))
+        how = dict(window=self.window, keep_first=self.keep_first, gate=g, out=o)
+        if plan.decode:
+            o = K.attention_window_decode(q, rows, plan, self.kv_heads, self.scale, fresh=kv if self.own_kv else None, **how)
+        else:
+            if self.own_kv:
+                K.scatter_rows(kv, plan.rows, rows.view(-1, self.cache_width))
+            o = K.attention_window(q, rows, plan, self.kv_heads, self.scale, **how)
+        return o.flatten(1) if out is None else out
