@@ -131,7 +131,7 @@ __global__ __launch_bounds__(WD_THREADS) void attn_window_decode_kernel(WdArgs a
         for (int j = 0; j < 8; ++j) acc[h][j] = fmaf(w, (float)vf[p][j], acc[h][j]);
       }
     }
-    if (fresh && hb == 0 && k0 + WD_KEYS >= vis.n) {       // the round that holds the newest key
+    if (fresh && hb == 0 && r1 == vis.n && k0 + WD_KEYS >= r1) {       // the round that holds the newest key
 #pragma unroll
       for (int p = 0; p < NP; ++p)
         if (k0 + p * KPP + g == vis.n - 1) {
