@@ -687,11 +687,11 @@ def parse_args(argv=None):
                     help="one of BASELINE.json's other configurations, counted from 1 (1 scan only, 2 256 frames, "
                          "3 2 048 frames + TransV + pdrop, 5 Qwen2.5 + dual encoder + fp8 attention), or `decode` (one "
                          "generated token against a 2 048-frame prefill cache); default: the headline run (10 240 "
-                         "frames); 4 is the headline run with --gpus 8; `fasovik`: prefill and decode of the Fasovik design at "
-                         "model-like layer sizes beside the hybrid Nemotron stack (--sizes, --prompt, --batch)")
-    ap.add_argument("--sizes", default="2k,4k", help="--config fasovik: layer sizes, of 2k and 4k (width), with commas between them")
-    ap.add_argument("--prompt", type=int, default=8192, help="--config fasovik: prompt tokens (and tokens in the cache of a decode step)")
-    ap.add_argument("--batch", type=int, default=4, help="--config fasovik: sequences of the batched decode step")
+                         "frames); 4 is the headline run with --gpus 8; `fasovik`, `fogorax`: prefill and decode of these designs "
+                         "at model-like layer sizes beside the Nemotron stack (--sizes, --prompt, --batch)")
+    ap.add_argument("--sizes", default="2k,4k", help="--config fasovik / fogorax: layer sizes, of 2k and 4k (width), with commas between them")
+    ap.add_argument("--prompt", type=int, default=8192, help="--config fasovik / fogorax: prompt tokens (and tokens in the cache of a decode step)")
+    ap.add_argument("--batch", type=int, default=4, help="--config fasovik / fogorax: sequences of the batched decode step")
     return ap.parse_args(argv)
 
 
@@ -699,13 +699,13 @@ def main():
     args = parse_args()
     if args.config == "decode":
         return config_decode(args)
-    if args.config == "fasovik":
+    if args.config in ("fasovik", "fogorax"):
         from timeviper_amd.devtools import bench_layers
         return bench_layers.main(args)
     try:
         args.config = int(args.config)
     except ValueError:
-        sys.exit("bench.py: --config takes 1, 2, 3, 4, 5, decode or fasovik")
+        sys.exit("bench.py: --config takes 1, 2, 3, 4, 5, decode, fasovik or fogorax")
     if args.config == 1:
         return config1_scan(args)
     if args.config == 2:
@@ -718,7 +718,7 @@ def main():
         sys.exit(subprocess.run([sys.executable, str(ROOT / "timeviper_amd" / "devtools" / "run_config5.py"), "4096",
                                  str(max(args.steps, 1)), "1"], cwd=str(ROOT)).returncode)
     elif args.config not in (0, 4):
-        sys.exit("bench.py: --config takes 1, 2, 3, 4, 5, decode or fasovik")
+        sys.exit("bench.py: --config takes 1, 2, 3, 4, 5, decode, fasovik or fogorax")
 
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(launch_children(__file__, sys.argv[1:], args.gpus))

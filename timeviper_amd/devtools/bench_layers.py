@@ -1,8 +1,10 @@
-"""Prefill and decode throughput of the Fasovik design at sizes that resemble a real model's layers, beside the hybrid Nemotron
-stack at the same width (bench.py --config fasovik).
+"""Prefill and decode throughput of the layer-list designs at sizes that resemble a real model's layers, beside the Nemotron
+stack at the same width (bench.py --config fasovik | fogorax).
 
-Both models get the same number of mixers of each kind (half attention, half recurrence), the same heads x 128 attention,
-recurrences of the same inner width and feed-forwards with the same number of active parameters per token; random weights.
+Fasovik: both models get the same number of mixers of each kind (half attention, half recurrence), the same heads x 128 attention,
+recurrences of the same inner width and feed-forwards with the same number of active parameters per token.  Fogorax: the other
+model is a stack of attention (same heads x 128, all keys visible) and MLP layers whose hidden width makes the parameters per
+layer the same.  Random weights.
 Per operator: the launches of one step, recorded with their arguments, run back to back between two events (decode: as a
 replayed graph), against the HBM roof (8 TB/s) or the dense bf16 MFMA roof (2.5 PFLOP/s) — whichever the algorithmic bytes /
 useful FLOPs of the launches make the slower."""
@@ -18,6 +20,10 @@ HBM, MFMA = 8000.0e9, 2500.0e12
 SIZES = {
     "2k": dict(width=2048, heads=16, rank=512, experts=64, identity=8, top=6, ff=1024, layers=8),
     "4k": dict(width=4096, heads=32, rank=512, experts=64, identity=8, top=8, ff=1536, layers=4),
+}
+FOGORAX_SIZES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, window=1024, keep=64, ff=5632, side=128, layers=8),
+    "4k": dict(width=4096, heads=32, kv_heads=8, window=4096, keep=16, ff=9216, side=256, layers=4),
 }
 
 
@@ -38,6 +44,27 @@ def nano_config(s):
                            num_hidden_layers=2 * s["layers"], hybrid_override_pattern="*-M-" * (s["layers"] // 2),
                            num_attention_heads=s["heads"], head_dim=128, num_key_value_heads=s["heads"], ssm_state_size=128,
                            mamba_num_heads=2 * s["heads"], mamba_head_dim=64, mamba_n_groups=8)
+
+
+def fogorax_config(s, positions):
+    """every second layer reads the keys and values of the one in front"""
+    from ..model.llm import FogoraxConfig
+    layers = []
+    for i in range(s["layers"]):
+        m = {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+             "mask": {"size": s["window"], "keep_first": s["keep"]}}
+        if i % 2:
+            m["kv_from"] = i - 1
+        layers.append({"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}})
+    return FogoraxConfig(vocab_size=32768, hidden_size=s["width"], layers=layers, side_dim=s["side"], max_positions=positions)
+
+
+def attention_stack_config(s):
+    """attention and MLP layers: two matrices of the MLP hold what the gate and the third matrix of a gated feed-forward do"""
+    from ..model.llm import NemotronHConfig
+    return NemotronHConfig(vocab_size=32768, hidden_size=s["width"], intermediate_size=(3 * s["ff"] + s["heads"] * 128) // 2,
+                           num_hidden_layers=2 * s["layers"], hybrid_override_pattern="*-" * s["layers"], num_attention_heads=s["heads"],
+                           head_dim=128, num_key_value_heads=s["kv_heads"])
 
 
 def build(cfg, dev):
@@ -75,6 +102,17 @@ def op_table(K):
         T, H, d, e = q.shape[-3], q.shape[-2], q.shape[-1], v.shape[-1]
         return T * (T + 1) * H * (d + e) * (q.shape[0] if q.dim() == 4 else 1), nb(q, k, v) + size(out)
 
+    def windowed(res, q, cache, plan, kv_heads, scale, window=K.NO_WINDOW, keep_first=0, **kw):
+        # visible pairs; q and o, and the rows of the cache that somebody sees
+        T, H, d = q.shape
+        e, pairs, seen = cache.shape[2] // kv_heads - d, 0, 0
+        for a, n in zip(plan.starts, plan.counts):
+            p = torch.arange(a, a + n, dtype=torch.float64)
+            lo = (p + 1 - window).clamp(min=0)
+            pairs += float((p + 1 - lo + lo.clamp(max=keep_first)).sum())
+            seen += a + n - int(lo[0]) + min(keep_first, int(lo[0]))
+        return 2 * pairs * H * (d + e), nb(q) + size(res) + seen * cache.shape[2] * 2
+
     def rows(offsets):
         return int(offsets[-1])
 
@@ -103,6 +141,15 @@ def op_table(K):
         "gemv_fused": lambda out, x, w, *a, **kw: (0, nb(w)),
         "selective_state_update": lambda out, st, *a, **kw: (0, 2 * nb(st)),
         "flash_attn_decode": lambda out, q, k, v, *a, **kw: (0, nb(k, v)),
+        "attention_window": windowed,
+        "attention_window_decode": lambda res, *a, **kw: (0, windowed(res, *a, **kw)[1]),
+        "norm_shift": lambda out, x, gain, eps, pending=None, *a, **kw: (0, nb(x, pending) + nb(*(t for t in out if t is not x))),
+        "residual_add": lambda out, x, u: (0, nb(x, u) + size(out)),
+        "gated_mul": lambda res, a, b, *r, **kw: (0, 3 * nb(a)),
+        "scatter_rows": lambda out, src, *a: (0, 2 * nb(src)),
+        "embed_scaled": lambda out, ids, *a, **kw: (0, size(out) + size(out) // 3),
+        "gemv_shift": lambda out, x, gain, eps, shift, state, plan, w, *a: (0, nb(w)),
+        "gemv_glu": lambda out, x, z, u, w, *a, **kw: (0, nb(w)),
         "latent_decode": lambda out, q, uk, uv, lat, keys, slot, *a, **kw: (0, nb(uk, uv) + int(keys.sum()) * lat.shape[2] * 2),
         "gemv_post": lambda out, x, w, *a, **kw: (0, nb(w)),
         # (every choice streams its expert's matrices; the router's weights are the product in front of it)
@@ -224,18 +271,21 @@ def main(args):
     out = {}
     T, batch = args.prompt, args.batch
     steps, warm = max(args.steps, 3), max(args.warmup, 2)
+    design = args.config
     for name in args.sizes.split(","):
-        s = SIZES[name]
+        s = (SIZES if design == "fasovik" else FOGORAX_SIZES)[name]
         out[name] = {"size": s}
-        for kind, cfg in (("fasovik", fasovik_config(s)), ("nemotron_hybrid", nano_config(s))):
+        pair = ((("fasovik", fasovik_config(s)), ("nemotron_hybrid", nano_config(s))) if design == "fasovik" else
+                (("fogorax", fogorax_config(s, T + 256)), ("nemotron_attention", attention_stack_config(s))))
+        for kind, cfg in pair:
             llm = build(cfg, dev)
             out[name][kind] = measure(llm, T, batch, steps, warm)
             del llm
             torch.cuda.empty_cache()
     first = next(iter(out))
-    f = out[first]["fasovik"]
+    f = out[first][design]
     print(json.dumps({
-        "metric": f"prefill tokens/s, Fasovik layers at width {SIZES[first]['width']}, one prompt", "value": f["prefill_tokens_per_s"],
+        "metric": f"prefill tokens/s, {design.capitalize()} layers at width {out[first]['size']['width']}, one prompt", "value": f["prefill_tokens_per_s"],
         "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": warm, "ms_per_step": f["prefill_ms"], "higher_is_better": True,
         "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
         "config": {"prompt_tokens": T, "decode_batches": sorted({1, batch}), "weights": "random init, seed 0"}, "sizes": out}), flush=True)
