@@ -546,7 +546,8 @@ int tv_embed_scaled_fwd(const int64_t* ids, const void* table, float* x, void* h
  *   h_before is the h of the previous row of the same sequence; of a sequence's first
  *   row: zeros at position 0, else row (position - 1) & 1 of the state block slot[b]
  *   ((2, D) fp32 blocks, state_stride floats apart); the last row's h goes to its row.
- *   Row t belongs to sequence seq[t], rows [cu[b], cu[b+1]), start[b] tokens in front.
+ *   Row t belongs to sequence seq[t], rows [cu[b], cu[b+1]), start[b] tokens in front
+ *   (single: every sequence has one row; seq and cu are not read).
  * tv_residual_add_fwd: x_out = x + u (fp32), h (optional) its rounding to dtype.
  * tv_gated_mul_fwd: o = f(a) * b[b_ids[row]] (b_ids NULL: b[row]; b has b_rows rows);
  *   act 0: f = sigmoid, 1: f = gelu (tanh form).
@@ -555,7 +556,8 @@ int tv_embed_scaled_fwd(const int64_t* ids, const void* table, float* x, void* h
  * --------------------------------------------------------------------- */
 int tv_norm_shift_fwd(const float* x, const void* y, const void* y_weight, float* x_out, const void* gain, const void* shift,
                       float* state, const int* seq, const int* cu, const int* start, const int* slot, void* h, void* hs,
-                      int64_t rows, int D, int64_t y_stride, int64_t state_stride, float eps, int dtype, void* stream);
+                      int64_t rows, int D, int64_t y_stride, int64_t state_stride, float eps, int single, int dtype,
+                      void* stream);
 int tv_residual_add_fwd(const float* x, const void* u, float* x_out, void* h, int64_t rows, int D, int64_t u_stride,
                         int dtype, void* stream);
 int tv_gated_mul_fwd(const void* a, const void* b, const int64_t* b_ids, void* o, int64_t rows, int cols, int64_t a_stride,
@@ -563,18 +565,18 @@ int tv_gated_mul_fwd(const void* a, const void* b, const int64_t* b_ids, void* o
 int tv_scatter_rows(const void* src, const int* rows_to, void* dst, int64_t rows, int cols, int64_t src_stride,
                     int64_t dst_stride, int dtype, void* stream);
 
-/* The same operators inside the matrix-vector products of a decode step (M = 1..4 bf16 rows, csrc/gemv.hip).
- * tv_gemv_shift_fwd: y[:, :n1] = hs W[:n1]^T, y[:, n1:] = h W[n1:]^T + bias, with x' / h / hs as tv_norm_shift_fwd
- *   computes them for one token per sequence (pending, pending_weight: its y and y_weight, or NULL).
- * tv_gemv_glu_fwd: y = [x | gelu(z) * u] W^T + bias, k1 columns of x; u rows by token id when u_ids.  With a residual
- *   (M, N) fp32: residual_out = residual + y (fp32) and h_out its bf16 rounding instead of y.                       */
-int tv_gemv_shift_fwd(const float* x, const void* pending, const void* pending_weight, float* x_out, const void* gain,
-                      const void* shift, float* state, const int* start, const int* slot, const void* W, const void* bias,
-                      void* y, int M, int N, int n1, int K, int64_t pending_stride, int64_t state_stride, int64_t ldw,
-                      int64_t y_stride, float eps, void* stream);
-int tv_gemv_glu_fwd(const void* x, const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W,
-                    const void* bias, const float* residual, float* residual_out, void* h_out, void* y, int M, int N, int k1,
-                    int K, int64_t x_stride, int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream);
+/* Matrix-vector products of a decode step's parallel layers (M = 1..4 bf16 rows, csrc/gemv.hip).
+ * tv_gemv_pair_fwd: y = x W[:n1]^T and act = gelu(x2 W[n1:n1+ff]^T + bias[:ff]) * (x2 W[n1+ff:]^T + bias[ff:])
+ *   (tanh form; ff 0: the first product alone).
+ * tv_gemv_add_fwd: residual_out = residual + x W^T + bias, (M, N) fp32 dense, and h_out (optional) its bf16 rounding.
+ * tv_gemv_glu_fwd: y = (gelu(z) * u) W^T, u (u_rows rows) by token id when u_ids.                                  */
+int tv_gemv_pair_fwd(const void* x, const void* x2, const void* W, const void* bias, void* y, void* act, int M, int n1, int ff,
+                     int K, int64_t x_stride, int64_t x2_stride, int64_t ldw, int64_t y_stride, int64_t act_stride,
+                     void* stream);
+int tv_gemv_add_fwd(const void* x, const void* W, const void* bias, const float* residual, float* residual_out, void* h_out,
+                    int M, int N, int K, int64_t x_stride, int64_t ldw, void* stream);
+int tv_gemv_glu_fwd(const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W, void* y, int M, int N,
+                    int K, int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream);
 
 /* ------------------------------------------------------------------------
  * Linear attention with one constant decay per head, ragged batches:

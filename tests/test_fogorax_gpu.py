@@ -147,7 +147,8 @@ def test_gated_products(dtype, n):
 
 
 # ------------------------------------------------------------------ attention in a window
-SHAPES = [(6, 3, 18, 22), (8, 2, 64, 96), (4, 4, 96, 40), (8, 4, 128, 128), (12, 1, 128, 64), (2, 1, 192, 256), (2, 2, 40, 8)]
+SHAPES = [(6, 3, 18, 22), (8, 2, 64, 96), (4, 4, 96, 40), (8, 4, 128, 128), (12, 1, 128, 64), (2, 1, 192, 256), (2, 2, 40, 8), (7, 1, 64, 128), (20, 1, 32, 24),
+          (10, 1, 128, 200)]
 
 
 def attention_case(H, G, d, e, starts, counts, capacity, dtype, seed=50):
@@ -266,52 +267,66 @@ def test_far_key_among_thousands():
 
 
 # ------------------------------------------------------------------ fused decode operators
-@pytest.mark.parametrize("M,D,n1,n2", [(1, 64, 24, 0), (2, 384, 70, 33), (4, 2048, 513, 512), (3, 4096, 64, 1), (1, 8192, 33, 40), (4, 4096, 100, 300)])
-@pytest.mark.parametrize("waits", [True, False])
-def test_matrix_vector_product_with_norm_and_shift_in_front(M, D, n1, n2, waits):
+@pytest.mark.parametrize("M,D,n1,ff", [(1, 64, 24, 0), (2, 384, 70, 33), (4, 2048, 513, 512), (3, 4096, 63, 1), (1, 8192, 33, 40), (4, 4096, 1, 3000),
+                                       (1, 9000, 5, 9), (2, 2056, 4097, 700), (1, 2048, 5120, 5632), (4, 2560, 3072, 6000)])
+def test_input_products_of_one_launch(M, D, n1, ff):
     from timeviper_amd import kernels as K
-    starts = dict(zip([2, 0, 4, 1][:M], [5, 0, 8, 1]))
-    x, y, gain, w, s, _ = shift_case(D, [1] * M, starts, BF, 80)
-    state = rnd((6, 2, D), 88, torch.float32)
-    weight, bias = rnd((n1 + n2, D), 86, BF, D ** -0.5), rnd((n2,), 87, BF)
-    c = cache_of([("state", (2, D))], 6, 32, BF, starts)
-    c.state(0).copy_(state)
-    plan = c.plan(list(starts), [1] * M)
-    x1, p = K.gemv_shift(x.to(DEV), gain.to(DEV), 1e-5, s.to(DEV), c.state(0), plan, weight.to(DEV), n1, bias.to(DEV) if n2 else None,
-                         *((y.to(DEV), w.to(DEV)) if waits else (None, None)))
-    xs = x.double() + (O.rms(y.double(), 1e-5) * w.double() if waits else 0)
-    h = O.norm_scalar(xs, gain.double(), 1e-5)
-    front = torch.stack([state[b, (st - 1) & 1].double() if st else torch.zeros(D).double() for b, st in starts.items()])
-    hs = h + (front - h) * s.double()
-    close(x1, xs, 2e-6)
-    close(p, torch.cat([hs @ weight[:n1].double().T, h @ weight[n1:].double().T + bias.double()], 1), 1e-2)
-    new = state.double()
-    for m, (b, st) in enumerate(starts.items()):
-        new[b, st & 1] = h[m]
-    close(c.state(0), new, 2e-6)
+    x, x2 = rnd((M, D), 80, BF), rnd((M, D), 81, BF)
+    weight, bias = rnd((n1 + 2 * ff, D), 86, BF, D ** -0.5), rnd((2 * ff,), 87, BF)
+    u = torch.zeros((M, ff + 16), dtype=BF, device=DEV)
+    y = K.gemv_pair(x.to(DEV), x2.to(DEV), weight.to(DEV), n1, bias.to(DEV) if ff else None, act_out=u[:, 8:8 + ff])
+    close(y, x.double() @ weight[:n1].double().T, 1e-2)
+    if ff:
+        z, v = (x2.double() @ weight[n1:].double().T + bias.double()).split(ff, dim=1)
+        close(u[:, 8:8 + ff], O.gelu_tanh(z) * v, 1e-2)
+    assert float(u[:, :8].abs().max()) == 0 and float(u[:, 8 + ff:].abs().max()) == 0
 
 
-@pytest.mark.parametrize("M,k1,k2,N", [(1, 64, 72, 40), (2, 512, 0, 70), (4, 2048, 5632, 513), (1, 4096, 11008, 100), (3, 0, 24, 384), (4, 0, 256, 2048)])
-def test_matrix_vector_product_of_gated_columns(M, k1, k2, N):
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("D", [76, 384, 2048, 4096])
+def test_norm_and_token_shift_of_single_tokens(D, dtype):
+    """One row per sequence, first tokens among them, step after step on one plan; against the whole sequences."""
     from timeviper_amd import kernels as K
-    Kd = k1 + k2
-    x, zu, weight, bias = rnd((M, k1), 90, BF), rnd((M, 2 * k2), 91, BF, 2.0), rnd((N, Kd), 92, BF, Kd ** -0.5), rnd((N,), 93, BF)
-    z, u = zu.split(k2, dim=1) if k2 else (None, None)
-    res = rnd((M, N), 94, torch.float32)
-    dev = lambda t: None if t is None else t.to(DEV)
-    zud = zu.to(DEV)
-    zd, ud = zud.split(k2, dim=1) if k2 else (None, None)
-    r = lambda t: t.to(BF).double()
-    f = torch.cat([x.double()] + ([r(O.gelu_tanh(z.double()) * u.double())] if k2 else []), 1)
-    want = f @ weight.double().T + bias.double()
-    close(K.gemv_glu(dev(x) if k1 else None, zd, ud, dev(weight), dev(bias)), want, 1e-2)
-    xs, hs = K.gemv_glu(dev(x) if k1 else None, zd, ud, dev(weight), dev(bias), residual=dev(res))
-    close(xs, res.double() + want, 2e-3)
-    assert torch.equal(hs, xs.to(BF))
-    if k2:
-        table, ids = rnd((9, k2 * 2), 95, BF), torch.tensor([8, 0, 3, 3][:M])
-        got = K.gemv_glu(dev(x) if k1 else None, zd, dev(table)[:, k2:], dev(weight), ids=ids.to(DEV))
-        f = torch.cat([x.double(), r(O.gelu_tanh(z.double()) * table[ids, k2:].double())], 1)
+    starts, steps = {2: 0, 0: 3, 5: 0}, 7
+    c = cache_of([("state", (2, 2, D))], 6, 32, dtype, {})
+    gain, s, w = rnd((), 1, dtype) + 1.2, rnd((D,), 2, dtype, 0.5), rnd((D,), 3, dtype) + 1
+    gain = gain.to(dtype)
+    xs = {b: rnd((n + steps, D), 10 + b, torch.float32) for b, n in starts.items()}
+    ys = {b: rnd((n + steps, D), 20 + b, dtype) for b, n in starts.items()}
+    run = lambda plan, x, y: K.norm_shift(x.to(DEV), gain.to(DEV), 1e-5, y.to(DEV), w.to(DEV), s.to(DEV), c.state(0)[:, 1], plan)
+    p = c.plan([0], [3])
+    run(p, xs[0][:3], ys[0][:3])
+    c.commit(p)
+    got = []
+    for t in range(steps):
+        p = c.plan(list(starts), [1] * 3)
+        got.append(run(p, *(torch.stack([v[b][n + t] for b, n in starts.items()]) for v in (xs, ys))))
+        c.commit(p)
+    for i, (b, n) in enumerate(starts.items()):
+        x = xs[b].double() + O.rms(ys[b].double(), 1e-5) * w.double()
+        h = O.norm_scalar(x, gain.double(), 1e-5)
+        for j, ref in ((0, x), (1, h), (2, O.token_shift(h, s.double()))):
+            close(torch.stack([g[j][i] for g in got]), ref[n:], 2e-6 if j == 0 else OP[dtype])
+
+
+@pytest.mark.parametrize("M,D,N", [(1, 64, 40), (2, 512, 70), (4, 7680, 513), (1, 7680, 2048), (1, 13312, 100), (4, 15104, 30), (3, 16384, 384)])
+def test_output_product_on_the_stream(M, D, N):
+    from timeviper_amd import kernels as K
+    x, weight, bias, res = rnd((M, D), 90, BF), rnd((N, D), 92, BF, D ** -0.5), rnd((N,), 93, BF), rnd((M, N), 94, torch.float32)
+    for b in (bias, None):
+        xs, hs = K.gemv_add(x.to(DEV), weight.to(DEV), res.to(DEV), None if b is None else b.to(DEV))
+        close(xs, res.double() + x.double() @ weight.double().T + (0 if b is None else b.double()), 2e-6)
+        assert torch.equal(hs, xs.to(BF))
+
+
+@pytest.mark.parametrize("M,n,N", [(3, 24, 384), (4, 256, 2048), (1, 8, 64), (2, 128, 4096)])
+def test_product_of_token_rows(M, n, N):
+    from timeviper_amd import kernels as K
+    z, u, weight, table = rnd((M, n), 95, BF, 2.0), rnd((M, n), 96, BF), rnd((N, n), 97, BF, n ** -0.5), rnd((9, 3 * n), 98, BF)
+    ids = torch.tensor([8, 0, 3, 3][:M])
+    for rows, by, got in ((u, None, K.gemv_glu(z.to(DEV), u.to(DEV), weight.to(DEV))),
+                          (table[:, n:2 * n], ids, K.gemv_glu(z.to(DEV), table.to(DEV)[:, n:2 * n], weight.to(DEV), ids=ids.to(DEV)))):
+        f = (O.gelu_tanh(z.double()) * (rows if by is None else rows[by]).double()).to(BF).double()
         close(got, f @ weight.double().T, 1e-2)
 
 

@@ -73,12 +73,13 @@ SIGNATURES = {
     "tv_rmsnorm_ex_fwd": (_i, [_p] * 8 + [_l, _l, _i] + [_l] * 5 + [_f] * 3 + [_i] * 3 + [_p]),
     "tv_moe_combine_norm_fwd": (_i, [_p] * 3 + [_i] + [_p] * 4 + [_l, _i] + [_l] * 4 + [_f] * 3 + [_i] * 3 + [_p]),
     "tv_embed_scaled_fwd": (_i, [_p] * 4 + [_l, _i, _l, _f] + [_p] * 4 + [_l, _i, _p]),
-    "tv_norm_shift_fwd": (_i, [_p] * 13 + [_l, _i, _l, _l, _f, _i, _p]),
+    "tv_norm_shift_fwd": (_i, [_p] * 13 + [_l, _i, _l, _l, _f, _i, _i, _p]),
     "tv_residual_add_fwd": (_i, [_p] * 4 + [_l, _i, _l, _i, _p]),
     "tv_gated_mul_fwd": (_i, [_p] * 4 + [_l, _i] + [_l] * 4 + [_i, _i, _p]),
     "tv_scatter_rows": (_i, [_p] * 3 + [_l, _i, _l, _l, _i, _p]),
-    "tv_gemv_shift_fwd": (_i, [_p] * 12 + [_i] * 4 + [_l] * 4 + [_f, _p]),
-    "tv_gemv_glu_fwd": (_i, [_p] * 4 + [_l] + [_p] * 6 + [_i] * 4 + [_l] * 5 + [_p]),
+    "tv_gemv_pair_fwd": (_i, [_p] * 6 + [_i] * 4 + [_l] * 5 + [_p]),
+    "tv_gemv_add_fwd": (_i, [_p] * 6 + [_i] * 3 + [_l] * 2 + [_p]),
+    "tv_gemv_glu_fwd": (_i, [_p] * 3 + [_l] + [_p] * 2 + [_i] * 3 + [_l] * 4 + [_p]),
     "tv_lightning_workspace_bytes": (_z, [_i] * 6),
     "tv_lightning_fwd": (_i, [_p] * 8 + [_i, _i, _p, _z] + [_i] * 3 + [_l] * 4 + [_i, _i, _p]),
     "tv_attn_generic_fwd": (_i, [_p] * 8 + [_i, _l] + [_i] * 4 + [_l] * 10 + [_f] + [_i] * 3 + [_p, _l, _l, _i, _p]),

@@ -62,27 +62,6 @@ __device__ __forceinline__ void split_of(const DecArgs& a, int b, int& Lk, int& 
   if (chunk == 0) chunk = AD_STEP;
 }
 
-__device__ __forceinline__ float xor16_max(float x) {
-  const unsigned u = __float_as_uint(x);
-  const auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-  return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
-}
-__device__ __forceinline__ float xor32_max(float x) {
-  const unsigned u = __float_as_uint(x);
-  const auto r = __builtin_amdgcn_permlane32_swap(u, u, false, false);
-  return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
-}
-__device__ __forceinline__ float xor16_sum(float x) {
-  const unsigned u = __float_as_uint(x);
-  const auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
-}
-__device__ __forceinline__ float xor32_sum(float x) {
-  const unsigned u = __float_as_uint(x);
-  const auto r = __builtin_amdgcn_permlane32_swap(u, u, false, false);
-  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
-}
-
 __global__ __launch_bounds__(AD_NW * 64) void attn_decode_kernel(DecArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char ad_smem[];
   const int tid = threadIdx.x, lane = tid & 63;

@@ -17,19 +17,16 @@
 //   PRO_POSTNORM  x' = residual + mult * (x * rsqrt(mean(x^2) + eps)) * (w_offset + w), fp32 (written to `res_out`, its bf16
 //                 rounding to `h_out`, by work-group 0), f = bf16(x')    post-norm models: the norm of the sublayer in front
 //   PRO_NORMGATE  f = bf16(x * rsqrt(mean(x^2) + eps) * w * sigmoid(gate))     lightning attention's output norm and gate
-//   PRO_SHIFT     x' = residual + rms(x) * w (the norm of what waits, optional; fp32, to `res_out`), h = rms(x') * gain,
-//                 hs = h + (h_before - h) * shift with the h of the sequence's previous token from its state (the new one goes to
-//                 the state's other row): rows of W below N1 meet bf16(hs), the others bf16(h) and a bias
-//   PRO_GLU       f = [x | bf16(gelu_tanh(z) * u)]: columns below K1 are x, the others a gated product, u's rows optionally
-//                 gathered by token id; epilogue: y + bias + residual in fp32 (`res_out`, `h_out`) when there is a residual
-// (the last four belong to models on a 32-bit residual stream and agree with tv_rmsnorm_ex_fwd, tv_norm_shift_fwd and tv_gated_mul_fwd)
+//   PRO_GLU       f = bf16(gelu_tanh(x) * u), u's rows optionally gathered by token id: for products with a short K (done again in every
+//                 work-group, a long one costs more than it saves: there the activation is an epilogue, gemv_pair_kernel below)
+// (the last three belong to models on a 32-bit residual stream and agree with tv_rmsnorm_ex_fwd and tv_gated_mul_fwd)
 // with the rounding points of the stand-alone kernels (norms.hip), so the fused step and the unfused one agree to the
 // accumulation order of the dot products.  fp32 accumulation (v_dot2c_f32_bf16), one rounding of y.
 #include "ssd_common.hpp"
 
 namespace {
 
-enum { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_RELU2 = 2, PRO_GATED = 3, PRO_POSTNORM = 4, PRO_NORMGATE = 5, PRO_SHIFT = 6, PRO_GLU = 7 };
+enum { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_RELU2 = 2, PRO_GATED = 3, PRO_POSTNORM = 4, PRO_NORMGATE = 5, PRO_GLU = 6 };
 constexpr int GV_THREADS = 256;
 constexpr int GV_WAVES = GV_THREADS / 64;
 constexpr int GV_MAXM = 4;
@@ -48,21 +45,14 @@ struct GemvArgs {
   const bf16_t *conv_w, *conv_b;   // (channels, 4), (channels) or NULL
   int conv_lo, conv_hi;
   float* y32;                      // the outputs in fp32 instead of bf16 (router logits)
-  const float* res;                // PRO_POSTNORM
+  const float* res;                // PRO_POSTNORM; PRO_NONE: the outputs are added to it (fp32 res_out, bf16 h_out instead of y)
   float* res_out;
   bf16_t* h_out;
   float mult, woff;
-  // PRO_SHIFT: x waits in `delta` (or NULL), its norm weight in norm_w (bf16); rows of W below N1 meet hs
-  const bf16_t *gain, *shift;
-  float* state;                    // blocks of (2, K), `sst` floats apart; row p & 1: the h of position p
-  const int *start, *slot;
-  int64_t sst;
-  int N1;
   // PRO_GLU
-  int K1;
-  const bf16_t *z, *u;
+  const bf16_t* u;
   const int64_t* u_ids;
-  int64_t zs, us, u_rows;
+  int64_t us, u_rows;
 };
 
 // the 8 norm weights of one 16-byte piece of x: requested here (fp32 weights: two 16-byte loads, bf16: one), turned into
@@ -105,23 +95,48 @@ template <int PRO, typename F>
 __device__ __forceinline__ void gemv_prologue(const GemvArgs& a, bf16_t* fx, float* red, F&& after_loads) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int K = a.K, nv = K / 8;
+  if constexpr (PRO == PRO_NONE || PRO == PRO_RELU2 || PRO == PRO_GLU) {
+    // pieces of all rows in one sequence, U requests at a time, the first ones in front of W's
+    constexpr int U = 4;
+    const int P = a.M * nv;
+    for (int b0 = 0; b0 < P; b0 += U * GV_THREADS) {
+      bf16x8 v[U], w[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        if (b0 + u * GV_THREADS >= P) break;         // (lanes past the end request the last piece again: no branch around a load)
+        const int pc = min(b0 + u * GV_THREADS + tid, P - 1), m = a.M == 1 ? 0 : pc / nv, c = pc - m * nv;
+        v[u] = *(const bf16x8*)(a.x + (int64_t)m * a.xs + 8 * c);
+        if (PRO == PRO_GLU) {
+          const int64_t ur = a.u_ids ? a.u_ids[m] : m;      // (checked on the host; a bad id reads the table's edge)
+          w[u] = *(const bf16x8*)(a.u + min(max(ur, (int64_t)0), a.u_rows - 1) * a.us + 8 * c);
+        }
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      if (b0 == 0) after_loads();
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int pc = b0 + u * GV_THREADS + tid;
+        if (pc < P) {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            if (PRO == PRO_RELU2) {
+              const float r = fmaxf((float)v[u][j], 0.f);
+              v[u][j] = (bf16_t)(r * r);
+            }
+            if (PRO == PRO_GLU) v[u][j] = (bf16_t)(gelu_tanh_f((float)v[u][j]) * (float)w[u][j]);
+          }
+          *(bf16x8*)(fx + (int64_t)8 * pc) = v[u];
+        }
+      }
+    }
+    __syncthreads();
+    return;
+  }
   for (int m = 0; m < a.M; ++m) {
     const bf16_t* xr = a.x + (int64_t)m * a.xs;
     bf16_t* fr = fx + (int64_t)m * K;
-    if (PRO == PRO_NONE || PRO == PRO_RELU2) {
-      if (m == 0) after_loads();
-      for (int iv = tid; iv < nv; iv += GV_THREADS) {
-        bf16x8 v = *(const bf16x8*)(xr + 8 * iv);
-        if (PRO == PRO_RELU2) {
-#pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            const float r = fmaxf((float)v[j], 0.f);
-            v[j] = (bf16_t)(r * r);
-          }
-        }
-        *(bf16x8*)(fr + 8 * iv) = v;
-      }
-    } else if (PRO == PRO_RMSNORM) {
+    if (PRO == PRO_RMSNORM) {
       constexpr int MAXV = 4;                        // K <= 8 * 256 * 4 (launcher)
       float vals[MAXV][8];
       NormW wq[MAXV];                                // (the weights are requested with x, not behind the reduction)
@@ -235,111 +250,6 @@ __device__ __forceinline__ void gemv_prologue(const GemvArgs& a, bf16_t* fx, flo
             if (a.h_out) *(bf16x8*)(a.h_out + (int64_t)m * K + 8 * iv) = o;
           }
         }
-      }
-    } else if (PRO == PRO_SHIFT) {
-      constexpr int MAXV = 4;                        // K <= 8 * 256 * 4 (launcher)
-      const int st = a.start[m];
-      float* sr = a.state + (int64_t)a.slot[m] * a.sst;
-      const float *rr = a.res + (int64_t)m * K, *pr = sr + (int64_t)((st - 1) & 1) * K;
-      bf16x8 dq[MAXV], wq[MAXV], hq[MAXV];
-      f32x4 r0[MAXV], r1[MAXV], p0[MAXV], p1[MAXV];
-#pragma unroll
-      for (int k = 0; k < MAXV; ++k) {               // (lanes past the end request the last piece again: no branch around a load)
-        if (k * GV_THREADS >= nv) break;
-        const int iv = min(tid + k * GV_THREADS, nv - 1);
-        r0[k] = *(const f32x4*)(rr + 8 * iv);
-        r1[k] = *(const f32x4*)(rr + 8 * iv + 4);
-        if (a.delta) {
-          dq[k] = *(const bf16x8*)(a.delta + (int64_t)m * a.ds + 8 * iv);
-          wq[k] = *(const bf16x8*)((const bf16_t*)a.norm_w + 8 * iv);
-        }
-        hq[k] = *(const bf16x8*)(a.shift + 8 * iv);
-        p0[k] = *(const f32x4*)(pr + 8 * iv);
-        p1[k] = *(const f32x4*)(pr + 8 * iv + 4);
-      }
-      const float gain = (float)*a.gain;
-      __builtin_amdgcn_sched_barrier(0);
-      if (m == 0) after_loads();
-      __builtin_amdgcn_sched_barrier(0);
-      auto total = [&](float v) __attribute__((always_inline)) {
-        v = wave_sum(v);
-        __syncthreads();                             // (red is used again)
-        if (lane == 0) red[wave] = v;
-        __syncthreads();
-        float t = 0.f;
-#pragma unroll
-        for (int i = 0; i < GV_WAVES; ++i) t += red[i];
-        return t;
-      };
-      if (a.delta) {
-        float ssq = 0.f;
-#pragma unroll
-        for (int k = 0; k < MAXV; ++k)
-          if (tid + k * GV_THREADS < nv) {
-#pragma unroll
-            for (int j = 0; j < 8; ++j) ssq = fmaf((float)dq[k][j], (float)dq[k][j], ssq);
-          }
-        const float rstd = rsqrtf(total(ssq) / (float)K + a.eps);
-#pragma unroll
-        for (int k = 0; k < MAXV; ++k) {
-          const int iv = tid + k * GV_THREADS;
-          if (iv < nv) {
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-              r0[k][j] = fmaf((float)dq[k][j] * rstd, (float)wq[k][j], r0[k][j]);
-              r1[k][j] = fmaf((float)dq[k][4 + j] * rstd, (float)wq[k][4 + j], r1[k][j]);
-            }
-            if (blockIdx.x == 0) {
-              float* ro = a.res_out + (int64_t)m * K + 8 * iv;
-              *(f32x4*)ro = r0[k];
-              *(f32x4*)(ro + 4) = r1[k];
-            }
-          }
-        }
-      }
-      float ssq = 0.f;
-#pragma unroll
-      for (int k = 0; k < MAXV; ++k)
-        if (tid + k * GV_THREADS < nv) {
-#pragma unroll
-          for (int j = 0; j < 4; ++j) ssq = fmaf(r0[k][j], r0[k][j], fmaf(r1[k][j], r1[k][j], ssq));
-        }
-      const float rstd = rsqrtf(total(ssq) / (float)K + a.eps) * gain;
-      bf16_t* fh = fx + (int64_t)(a.M + m) * K;
-#pragma unroll
-      for (int k = 0; k < MAXV; ++k) {
-        const int iv = tid + k * GV_THREADS;
-        if (iv < nv) {
-          bf16x8 o, os;
-          r0[k] *= rstd;
-          r1[k] *= rstd;
-#pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            const float h = j < 4 ? r0[k][j & 3] : r1[k][j & 3], before = st > 0 ? (j < 4 ? p0[k][j & 3] : p1[k][j & 3]) : 0.f;
-            o[j] = (bf16_t)h;
-            os[j] = (bf16_t)fmaf(before - h, (float)hq[k][j], h);
-          }
-          *(bf16x8*)(fr + 8 * iv) = os;
-          *(bf16x8*)(fh + 8 * iv) = o;
-          if (blockIdx.x == 0) {                     // (the other row of the state: nobody reads it in this launch)
-            float* so = sr + (int64_t)(st & 1) * K + 8 * iv;
-            *(f32x4*)so = r0[k];
-            *(f32x4*)(so + 4) = r1[k];
-          }
-        }
-      }
-    } else if (PRO == PRO_GLU) {
-      if (m == 0) after_loads();
-      const int nv1 = a.K1 / 8;
-      for (int iv = tid; iv < nv1; iv += GV_THREADS) *(bf16x8*)(fr + 8 * iv) = *(const bf16x8*)(xr + 8 * iv);
-      const int64_t ur = a.u_ids ? a.u_ids[m] : m;
-      const bool ok = ur >= 0 && ur < a.u_rows;      // (callers check ids on the host; a bad one reads nothing)
-      for (int iv = tid; iv < nv - nv1; iv += GV_THREADS) {
-        const bf16x8 z = *(const bf16x8*)(a.z + (int64_t)m * a.zs + 8 * iv), zero = {};
-        bf16x8 u = ok ? *(const bf16x8*)(a.u + ur * a.us + 8 * iv) : zero;
-#pragma unroll
-        for (int j = 0; j < 8; ++j) u[j] = (bf16_t)(gelu_tanh_f((float)z[j]) * (float)u[j]);
-        *(bf16x8*)(fr + 8 * (nv1 + iv)) = u;
       }
     } else {                                         // PRO_GATED: a wave per group of `group` channels
       constexpr int MAXV = 4, GPW = 1;               // group <= 8 * 64 * 4 (launcher)
@@ -503,7 +413,7 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_bf16_kernel(GemvArgs a) {
           float sm = 0.f;
 #pragma unroll
           for (int w = 0; w < GV_WAVES; ++w) sm += part[par][j][w][r][m];
-          if (PRO == PRO_GLU && a.res) {
+          if (PRO == PRO_NONE && a.res) {
             const float v = sm + (a.bias ? (float)a.bias[n] : 0.f) + a.res[(int64_t)m * a.N + n];
             a.res_out[(int64_t)m * a.N + n] = v;
             if (a.h_out) a.h_out[(int64_t)m * a.N + n] = (bf16_t)v;
@@ -567,16 +477,10 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
 #pragma unroll
           for (int m = 0; m < MT; ++m)
             if (MT == 1 || m < a.M) {
-              // (PRO_SHIFT: hs for the rows below N1, h — behind it in LDS — for the others)
-              const int o0 = PRO == PRO_SHIFT && n0 >= a.N1 ? a.M * K : 0;
-              const bf16x8 xv = *(const bf16x8*)(fl + o0 + (int64_t)m * K + 512 * (i0 + u));
+              const bf16x8 xv = *(const bf16x8*)(fl + (int64_t)m * K + 512 * (i0 + u));
 #pragma unroll
               for (int r = 0; r < R; ++r)
-                if (n0 + r * TW < a.N) {
-                  if (PRO == PRO_SHIFT && o0 == 0 && n0 + r * TW >= a.N1)      // (wave uniform)
-                    acc[r][m] = dot8(w[u][r], *(const bf16x8*)(fl + (int64_t)(a.M + m) * K + 512 * (i0 + u)), acc[r][m]);
-                  else acc[r][m] = dot8(w[u][r], xv, acc[r][m]);
-                }
+                if (n0 + r * TW < a.N) acc[r][m] = dot8(w[u][r], xv, acc[r][m]);
             }
         }
     };
@@ -603,8 +507,7 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
 #pragma unroll
       for (int m = 0; m < MT; ++m) tot[r][m] = (MT == 1 || m < a.M) ? wave_total(acc[r][m]) : 0.f;
     if (lane < R && nmine < a.N) {
-      const int nb = PRO == PRO_SHIFT ? nmine - a.N1 : nmine;        // (PRO_SHIFT: the bias belongs to the rows from N1 on)
-      const float bs = a.bias && nb >= 0 ? (float)a.bias[nb] : 0.f;
+      const float bs = a.bias ? (float)a.bias[nmine] : 0.f;
 #pragma unroll
       for (int m = 0; m < MT; ++m)
         if (MT == 1 || m < a.M) {
@@ -629,13 +532,128 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_rows_kernel(GemvArgs a) {
             *(bf16x4*)st = win;
             out = (bf16_t)silu_f(acc_c);
           }
-          if (PRO == PRO_GLU && a.res) {
+          if (PRO == PRO_NONE && a.res) {
             v += bs + a.res[(int64_t)m * a.N + nmine];
             a.res_out[(int64_t)m * a.N + nmine] = v;
             if (a.h_out) a.h_out[(int64_t)m * a.N + nmine] = (bf16_t)v;
           } else if (a.y32) a.y32[(int64_t)m * a.ys + nmine] = v;
           else a.y[(int64_t)m * a.ys + nmine] = out;
         }
+    }
+  }
+}
+
+// ---------------------------------------------------------------- two products of one launch, activation in the epilogue
+// y = x W[:n1]^T and act = gelu_tanh(x2 Wg^T + bg) * (x2 Wu^T + bu), Wg = rows [n1, n1 + ff) of W, Wu = rows [n1 + ff, n1 + 2 ff): the input side
+// of a layer whose mixer and feed-forward run in parallel.  A wave takes rows in groups of two — two neighbours of the first
+// part, or the gate and up row of one output, which meet in its registers — GP groups at a time; a work-group serves one part
+// and holds that part's vector only.
+struct PairArgs {
+  const bf16_t *x, *x2, *W, *bias;
+  bf16_t *y, *act;
+  int M, n1, ff, K, wg1;                             // work-groups [0, wg1): the first part
+  int64_t xs, x2s, ldw, ys, as;
+};
+
+template <int MT, int GP, int NB, bool NT>
+__global__ __launch_bounds__(GV_THREADS) void gemv_pair_kernel(PairArgs a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char gv_smem[];
+  bf16_t* fx = (bf16_t*)gv_smem;                     // [M][K]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int K = a.K, nv = K / 8, nins = (nv + 63) / 64;
+  const bool glu = (int)blockIdx.x >= a.wg1;
+  const int NG = glu ? a.ff : (a.n1 + 1) / 2;
+  const int TW = (glu ? (int)gridDim.x - a.wg1 : a.wg1) * GV_WAVES;
+  const int gw = ((int)blockIdx.x - (glu ? a.wg1 : 0)) * GV_WAVES + wave;
+  // row r of group g; a group past the end, or the missing neighbour of the last one, repeats a row that exists (not stored)
+  auto row_of = [&](int g, int r) __attribute__((always_inline)) {
+    g = min(g, NG - 1);
+    return glu ? a.n1 + g + r * a.ff : min(2 * g + r, a.n1 - 1);
+  };
+  auto load_batch = [&](bf16x8 (&dst)[NB][GP][2], int g0, int i0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < GP; ++i)
+      if (g0 + i * TW < NG) {                        // (wave uniform)
+#pragma unroll
+        for (int r = 0; r < 2; ++r) {
+          const bf16_t* wp = a.W + (int64_t)row_of(g0 + i * TW, r) * a.ldw + 8 * lane;
+#pragma unroll
+          for (int u = 0; u < NB; ++u) {
+            const bf16x8 z = {};
+            dst[u][i][r] = 64 * (i0 + u) + lane < nv ? ldw8<NT>(wp + 512 * (i0 + u)) : z;
+          }
+        }
+      }
+  };
+  bf16x8 cur[NB][GP][2];
+  {
+    constexpr int U = 4;
+    const bf16_t* xp = glu ? a.x2 : a.x;
+    const int64_t xs = glu ? a.x2s : a.xs;
+    const int P = a.M * nv;
+    for (int b0 = 0; b0 < P; b0 += U * GV_THREADS) {
+      bf16x8 v[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        if (b0 + u * GV_THREADS >= P) break;
+        const int pc = min(b0 + u * GV_THREADS + tid, P - 1), m = MT == 1 ? 0 : pc / nv;
+        v[u] = *(const bf16x8*)(xp + (int64_t)m * xs + 8 * (pc - m * nv));
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      if (b0 == 0 && gw < NG) load_batch(cur, gw, 0);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int pc = b0 + u * GV_THREADS + tid;
+        if (pc < P) *(bf16x8*)(fx + (int64_t)8 * pc) = v[u];
+      }
+    }
+    __syncthreads();
+  }
+  const bf16_t* fl = fx + 8 * lane;
+  for (int g0 = gw; g0 < NG; g0 += GP * TW) {
+    float acc[GP][2][MT];
+#pragma unroll
+    for (int i = 0; i < GP; ++i)
+#pragma unroll
+      for (int m = 0; m < MT; ++m) acc[i][0][m] = acc[i][1][m] = 0.f;
+    for (int i0 = 0; i0 < nins; i0 += NB) {
+      if (g0 != gw || i0) load_batch(cur, g0, i0);
+#pragma unroll
+      for (int u = 0; u < NB; ++u)
+        if (64 * (i0 + u) + lane < nv) {
+#pragma unroll
+          for (int m = 0; m < MT; ++m)
+            if (MT == 1 || m < a.M) {
+              const bf16x8 xv = *(const bf16x8*)(fl + (int64_t)m * K + 512 * (i0 + u));
+#pragma unroll
+              for (int i = 0; i < GP; ++i)
+                if (g0 + i * TW < NG) {
+                  acc[i][0][m] = dot8(cur[u][i][0], xv, acc[i][0][m]);
+                  acc[i][1][m] = dot8(cur[u][i][1], xv, acc[i][1][m]);
+                }
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < GP; ++i) {
+      const int g = g0 + i * TW;
+      if (g < NG) {
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+          if (MT == 1 || m < a.M) {
+            const float p = wave_total(acc[i][0][m]), q = wave_total(acc[i][1][m]);
+            if (lane == 0) {
+              if (glu) {
+                const float z = p + (float)a.bias[g], u = q + (float)a.bias[a.ff + g];
+                a.act[(int64_t)m * a.as + g] = (bf16_t)(gelu_tanh_f(z) * u);
+              } else {
+                a.y[(int64_t)m * a.ys + 2 * g] = (bf16_t)p;
+                if (2 * g + 1 < a.n1) a.y[(int64_t)m * a.ys + 2 * g + 1] = (bf16_t)q;
+              }
+            }
+          }
+      }
     }
   }
 }
@@ -767,7 +785,12 @@ __global__ __launch_bounds__(GV_THREADS) void gemv_splitk_reg_kernel(GemvArgs a)
           float sm = 0.f;
 #pragma unroll
           for (int w = 0; w < GV_WAVES; ++w) sm += part[par][j][w][r];
-          a.y[n] = (bf16_t)(sm + (a.bias ? (float)a.bias[n] : 0.f));
+          sm += a.bias ? (float)a.bias[n] : 0.f;
+          if (PRO == PRO_NONE && a.res) {
+            sm += a.res[n];
+            a.res_out[n] = sm;
+            if (a.h_out) a.h_out[n] = (bf16_t)sm;
+          } else a.y[n] = (bf16_t)sm;
         }
       }
       par ^= 1; gi = 0; nflush = n0 + R * G;
@@ -808,7 +831,7 @@ int launch_gemv_r(const GemvArgs& a, hipStream_t st) {
 }
 template <int PRO, int MT, bool NT, int R, int NB>
 int launch_gemv_rows(const GemvArgs& a, hipStream_t st) {
-  const size_t lds = (size_t)(PRO == PRO_SHIFT ? 2 : 1) * a.M * a.K * sizeof(bf16_t);
+  const size_t lds = (size_t)a.M * a.K * sizeof(bf16_t);
   static const hipError_t attr = hipFuncSetAttribute((const void*)gemv_rows_kernel<PRO, MT, NT, R, NB>,
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
   if (attr != hipSuccess) {
@@ -845,13 +868,14 @@ bool reg_takes(const GemvArgs& a) {
 template <int PRO, int MT>
 int launch_gemv_m(const GemvArgs& a, hipStream_t st) {
   static const int force = [] { const char* e = getenv("TV_GEMV_SPLITK"); return e ? atoi(e) : -1; }();    // (dev: 0 / 1)
-  const bool splitk = a.conv_state ? false : (force >= 0 ? force != 0 : a.K >= 8192);
+  // (few long rows: a row per wave would leave half of the waves idle)
+  const bool few = PRO == PRO_NONE && a.K >= 4096 && a.N <= 2 * GV_WAVES * gemv_wgs() * cu_count();
+  const bool splitk = a.conv_state ? false : (force >= 0 ? force != 0 : a.K >= 8192 || few);
   if constexpr (MT == 1 && (PRO == PRO_NONE || PRO == PRO_RELU2 || PRO == PRO_GATED)) {
     if (splitk && !a.y32 && reg_takes<PRO>(a)) return gemv_nt() ? launch_splitk_reg<PRO, true>(a, st) : launch_splitk_reg<PRO, false>(a, st);
   }
   // (the gated prologue holds two groups' operands in registers: no second set of W rows beside them)
   constexpr bool PF = PRO != PRO_GATED;
-  if constexpr (PRO == PRO_SHIFT) return gemv_nt() ? launch_gemv_rows<PRO, MT, true, 2, 10>(a, st) : launch_gemv_rows<PRO, MT, false, 2, 10>(a, st);
   if (!gemv_nt()) return splitk ? launch_gemv_r<PRO, MT, 2, 8, false, PF>(a, st) : launch_gemv_rows<PRO, MT, false, 2, 10>(a, st);
   return splitk ? launch_gemv_r<PRO, MT, 2, 8, true, PF>(a, st) : launch_gemv_rows<PRO, MT, true, 2, 10>(a, st);
 }
@@ -918,6 +942,7 @@ extern "C" int tv_gemv_post_fwd(const void* x, const void* W, void* y, int y_dty
                                 const void* norm_weight, int norm_weight_dtype, float weight_offset, float mult, float eps,
                                 const void* gate, int64_t gate_stride, void* stream) {
   TV_CHECK_ARG(x && W && y, "gemv_post: null pointer");
+  TV_CHECK_ARG(prologue == PRO_POSTNORM || !residual, "gemv_post: a residual belongs to prologue 4 (tv_gemv_add_fwd adds the outputs to one)");
   TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8, "gemv_post: M %d must be 1..%d, N %d >= 1, K %d >= 8", M, GV_MAXM, N, K);
   TV_CHECK_ARG(y_dtype == TV_BF16 || y_dtype == TV_F32, "gemv_post: y dtype %d", y_dtype);
   TV_CHECK_ARG(prologue == PRO_NONE || prologue == PRO_POSTNORM || prologue == PRO_NORMGATE, "gemv_post: prologue %d", prologue);
@@ -944,43 +969,71 @@ extern "C" int tv_gemv_post_fwd(const void* x, const void* W, void* y, int y_dty
   return launch_gemv<PRO_NORMGATE>(a, st);
 }
 
-// The product in front of a parallel layer's sublayers: rows of W below n1 read the shifted h, the others h (and a bias).
-extern "C" int tv_gemv_shift_fwd(const float* x, const void* pending, const void* pending_weight, float* x_out, const void* gain,
-                                 const void* shift, float* state, const int* start, const int* slot, const void* W, const void* bias,
-                                 void* y, int M, int N, int n1, int K, int64_t pending_stride, int64_t state_stride, int64_t ldw,
-                                 int64_t y_stride, float eps, void* stream) {
-  TV_CHECK_ARG(x && gain && shift && state && start && slot && W && y, "gemv_shift: null pointer");
-  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8 && n1 >= 0 && n1 <= N, "gemv_shift: M %d must be 1..%d, N %d >= 1, K %d >= 8", M, GV_MAXM, N, K);
-  TV_CHECK_ARG(!pending || (pending_weight && x_out && x_out != x), "gemv_shift: what waits needs its weight and a stream to be written (not in place)");
-  if (K % 8 || ldw % 8 || pending_stride % 8 || state_stride % 4 || ((uintptr_t)x & 15) || ((uintptr_t)pending & 15) || ((uintptr_t)pending_weight & 15) ||
-      ((uintptr_t)x_out & 15) || ((uintptr_t)shift & 15) || ((uintptr_t)state & 15) || ((uintptr_t)W & 15))
-    TV_UNSUPPORTED("gemv_shift: K and the row strides must be multiples of 8 elements, operands 16-byte aligned");
-  if ((size_t)2 * M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_shift: 2 x M x K = 2 x %d x %d does not fit the 128 KiB of LDS", M, K);
-  if (K > 8 * GV_THREADS * 4) TV_UNSUPPORTED("gemv_shift: rows of <= %d channels", 8 * GV_THREADS * 4);
+// residual + x W^T + bias in fp32 (residual_out) and its bf16 rounding (h_out): the output side of a layer on a 32-bit stream.
+extern "C" int tv_gemv_add_fwd(const void* x, const void* W, const void* bias, const float* residual, float* residual_out, void* h_out, int M,
+                               int N, int K, int64_t x_stride, int64_t ldw, void* stream) {
+  TV_CHECK_ARG(x && W && residual && residual_out, "gemv_add: null pointer");
+  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8, "gemv_add: M %d must be 1..%d, N %d >= 1, K %d >= 8", M, GV_MAXM, N, K);
+  if (K % 8 || ldw % 8 || x_stride % 8 || ((uintptr_t)x & 15) || ((uintptr_t)W & 15))
+    TV_UNSUPPORTED("gemv_add: K and the row strides must be multiples of 8 elements, operands 16-byte aligned");
+  if ((size_t)M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_add: M x K = %d x %d does not fit the 128 KiB of LDS x is held in", M, K);
   GemvArgs a{};
-  a.W = (const bf16_t*)W; a.bias = (const bf16_t*)bias; a.y = (bf16_t*)y;
-  a.M = M; a.N = N; a.K = K; a.group = K; a.ldw = ldw; a.ys = y_stride; a.eps = eps;
-  a.res = x; a.res_out = x_out; a.delta = (const bf16_t*)pending; a.ds = pending_stride; a.norm_w = pending_weight;
-  a.gain = (const bf16_t*)gain; a.shift = (const bf16_t*)shift; a.state = state; a.sst = state_stride; a.start = start; a.slot = slot;
-  a.N1 = n1;
-  return launch_gemv<PRO_SHIFT>(a, (hipStream_t)stream);
+  a.x = (const bf16_t*)x; a.W = (const bf16_t*)W; a.bias = (const bf16_t*)bias;
+  a.M = M; a.N = N; a.K = K; a.group = K; a.xs = x_stride; a.ldw = ldw; a.ys = N;
+  a.res = residual; a.res_out = residual_out; a.h_out = (bf16_t*)h_out;
+  return launch_gemv<PRO_NONE>(a, (hipStream_t)stream);
 }
 
-// y = [x | gelu_tanh(z) u] W^T (+ bias); with a residual: residual + y in fp32 (and its bf16 rounding) instead of y.
-extern "C" int tv_gemv_glu_fwd(const void* x, const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W,
-                               const void* bias, const float* residual, float* residual_out, void* h_out, void* y, int M, int N, int k1,
-                               int K, int64_t x_stride, int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream) {
-  TV_CHECK_ARG(W && (x || k1 == 0) && ((z && u) || k1 == K) && (residual ? residual_out != nullptr : y != nullptr), "gemv_glu: null pointer");
-  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8 && k1 >= 0 && k1 <= K && (k1 == K || u_rows > 0),
-               "gemv_glu: M %d must be 1..%d, N %d >= 1, K %d >= 8, %d columns of x", M, GV_MAXM, N, K, k1);
-  if (K % 8 || k1 % 8 || ldw % 8 || x_stride % 8 || z_stride % 8 || u_stride % 8 || ((uintptr_t)x & 15) || ((uintptr_t)z & 15) ||
-      ((uintptr_t)u & 15) || ((uintptr_t)W & 15))
-    TV_UNSUPPORTED("gemv_glu: K, its parts and the row strides must be multiples of 8 elements, operands 16-byte aligned");
+// y = (gelu_tanh(z) u) W^T, u's rows by token id when u_ids.
+extern "C" int tv_gemv_glu_fwd(const void* z, const void* u, const int64_t* u_ids, int64_t u_rows, const void* W, void* y, int M, int N, int K,
+                               int64_t z_stride, int64_t u_stride, int64_t ldw, int64_t y_stride, void* stream) {
+  TV_CHECK_ARG(z && u && W && y && u_rows > 0, "gemv_glu: null pointer");
+  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && N >= 1 && K >= 8, "gemv_glu: M %d must be 1..%d, N %d >= 1, K %d >= 8", M, GV_MAXM, N, K);
+  if (K % 8 || ldw % 8 || z_stride % 8 || u_stride % 8 || ((uintptr_t)z & 15) || ((uintptr_t)u & 15) || ((uintptr_t)W & 15))
+    TV_UNSUPPORTED("gemv_glu: K and the row strides must be multiples of 8 elements, operands 16-byte aligned");
   if ((size_t)M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_glu: M x K = %d x %d does not fit the 128 KiB of LDS f(x) is held in", M, K);
   GemvArgs a{};
-  a.x = (const bf16_t*)x; a.W = (const bf16_t*)W; a.bias = (const bf16_t*)bias; a.y = (bf16_t*)y;
-  a.M = M; a.N = N; a.K = K; a.group = K; a.xs = x_stride; a.ldw = ldw; a.ys = y_stride;
-  a.res = residual; a.res_out = residual_out; a.h_out = (bf16_t*)h_out;
-  a.K1 = k1; a.z = (const bf16_t*)z; a.u = (const bf16_t*)u; a.u_ids = u_ids; a.zs = z_stride; a.us = u_stride; a.u_rows = u_rows;
+  a.x = (const bf16_t*)z; a.W = (const bf16_t*)W; a.y = (bf16_t*)y;
+  a.M = M; a.N = N; a.K = K; a.group = K; a.xs = z_stride; a.ldw = ldw; a.ys = y_stride;
+  a.u = (const bf16_t*)u; a.u_ids = u_ids; a.us = u_stride; a.u_rows = u_rows;
   return launch_gemv<PRO_GLU>(a, (hipStream_t)stream);
+}
+
+template <int MT, int GP, int NB>
+static int launch_pair(const PairArgs& a, int wgs, hipStream_t st) {
+  const size_t lds = (size_t)a.M * a.K * sizeof(bf16_t);
+  static const hipError_t attr = hipFuncSetAttribute((const void*)gemv_pair_kernel<MT, GP, NB, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
+  if (attr != hipSuccess) {
+    tv_set_error("gemv_pair: cannot reserve 128 KiB of LDS: %s", hipGetErrorString(attr));
+    return TV_ERR_LAUNCH;
+  }
+  gemv_pair_kernel<MT, GP, NB, true><<<dim3((unsigned)wgs), GV_THREADS, lds, st>>>(a);
+  TV_LAUNCH_CHECK();
+}
+
+// y = x W[:n1]^T and act = gelu_tanh(x2 W[n1 : n1 + ff]^T + bias[:ff]) * (x2 W[n1 + ff :]^T + bias[ff:]).
+extern "C" int tv_gemv_pair_fwd(const void* x, const void* x2, const void* W, const void* bias, void* y, void* act, int M, int n1, int ff, int K,
+                                int64_t x_stride, int64_t x2_stride, int64_t ldw, int64_t y_stride, int64_t act_stride, void* stream) {
+  TV_CHECK_ARG(x && W && y && (ff == 0 || (x2 && bias && act)), "gemv_pair: null pointer");
+  TV_CHECK_ARG(M >= 1 && M <= GV_MAXM && n1 >= 1 && ff >= 0 && K >= 8, "gemv_pair: M %d must be 1..%d, rows %d + 2 x %d, K %d >= 8", M, GV_MAXM, n1, ff, K);
+  if (K % 8 || ldw % 8 || x_stride % 8 || x2_stride % 8 || ((uintptr_t)x & 15) || ((uintptr_t)x2 & 15) || ((uintptr_t)W & 15))
+    TV_UNSUPPORTED("gemv_pair: K and the row strides must be multiples of 8 elements, operands 16-byte aligned");
+  if ((size_t)M * K * 2 > 128 * 1024) TV_UNSUPPORTED("gemv_pair: M x K = %d x %d does not fit the 128 KiB of LDS", M, K);
+  PairArgs a{(const bf16_t*)x, (const bf16_t*)x2, (const bf16_t*)W, (const bf16_t*)bias, (bf16_t*)y, (bf16_t*)act, M, n1, ff, K, 0,
+             x_stride, x2_stride, ldw, y_stride, act_stride};
+  // two work-groups per CU, shared out by rows; no more than there are groups for the waves
+  const int most = gemv_wgs() * cu_count(), g1 = (n1 + 1) / 2, need1 = (g1 + GV_WAVES - 1) / GV_WAVES, need2 = (ff + GV_WAVES - 1) / GV_WAVES;
+  int w1 = need1, w2 = need2;
+  if (w1 + w2 > most) {
+    w1 = (int)((int64_t)most * g1 / (g1 + ff));
+    w1 = w1 < 1 ? 1 : w1 > most - (ff ? 1 : 0) ? most - (ff ? 1 : 0) : w1;
+    w2 = ff ? most - w1 : 0;
+    w1 = w1 > need1 ? need1 : w1;
+    w2 = w2 > need2 ? need2 : w2;
+  }
+  a.wg1 = w1;
+  hipStream_t st = (hipStream_t)stream;
+  // short rows: two groups at a time keep as many loads in flight as one group of long rows
+  if (K <= 2560) return M == 1 ? launch_pair<1, 2, 5>(a, w1 + w2, st) : launch_pair<GV_MAXM, 2, 5>(a, w1 + w2, st);
+  return M == 1 ? launch_pair<1, 1, 10>(a, w1 + w2, st) : launch_pair<GV_MAXM, 1, 10>(a, w1 + w2, st);
 }

@@ -50,7 +50,7 @@ struct NsArgs {
   float* state;            // (slots, 2, D) blocks, `ss` floats apart
   const int *seq, *cu, *start, *slot;
   void *h, *hs;
-  int rows, D, run;
+  int rows, D, run, single;          // single: one row per sequence
   int64_t ys, ss;
   float eps;
 };
@@ -138,8 +138,8 @@ __global__ __launch_bounds__(SO_THREADS) void norm_shift_kernel(NsArgs a) {
     bool first = false;
     int b = 0, st = 0;
     if (a.shift) {
-      b = a.seq[t];
-      first = t == a.cu[b];
+      b = a.single ? t : a.seq[t];
+      first = a.single || t == a.cu[b];
       if (first) {
         st = a.start[b];
         const float* sr = a.state + (int64_t)a.slot[b] * a.ss + (int64_t)((st - 1) & 1) * a.D;
@@ -169,7 +169,7 @@ __global__ __launch_bounds__(SO_THREADS) void norm_shift_kernel(NsArgs a) {
       }
     }
     if (first) {
-      const int last = a.cu[b + 1] - 1, p = st + last - t;
+      const int last = a.single ? t : a.cu[b + 1] - 1, p = st + last - t;
       if (last == t) {
         put_state(cur, b, p);
       } else {
@@ -331,13 +331,13 @@ bool fits(int64_t n) { return n < (1ll << 31); }
 
 extern "C" int tv_norm_shift_fwd(const float* x, const void* y, const void* y_weight, float* x_out, const void* gain, const void* shift,
                                  float* state, const int* seq, const int* cu, const int* start, const int* slot, void* h, void* hs,
-                                 int64_t rows, int D, int64_t y_stride, int64_t state_stride, float eps, int dtype, void* stream) {
+                                 int64_t rows, int D, int64_t y_stride, int64_t state_stride, float eps, int single, int dtype, void* stream) {
   TV_CHECK_ARG(rows >= 0 && fits(rows) && D > 0, "norm_shift: bad sizes");
   if (rows == 0) return TV_OK;
   TV_CHECK_ARG(x && gain && (h || hs) && (!y || y_weight) && (!x_out || y), "norm_shift: null pointer");
   TV_CHECK_ARG(!shift || (state && seq && cu && start && slot && hs), "norm_shift: the token shift needs its state and the plan of the step");
   TV_CHECK_ARG(x_out != x, "norm_shift: x is not updated in place (rows are read by their neighbours)");
-  NsArgs a{x, y, y_weight, x_out, gain, shift, state, seq, cu, start, slot, h, hs, (int)rows, D, 1, y_stride, state_stride, eps};
+  NsArgs a{x, y, y_weight, x_out, gain, shift, state, seq, cu, start, slot, h, hs, (int)rows, D, 1, single, y_stride, state_stride, eps};
   if (dtype == TV_F32) return norm_shift<float>(a, (hipStream_t)stream);
   if (dtype == TV_BF16) return norm_shift<bf16_t>(a, (hipStream_t)stream);
   TV_UNSUPPORTED("norm_shift: dtype %d", dtype);

@@ -148,8 +148,9 @@ def op_table(K):
         "gated_mul": lambda res, a, b, *r, **kw: (0, 3 * nb(a)),
         "scatter_rows": lambda out, src, *a: (0, 2 * nb(src)),
         "embed_scaled": lambda out, ids, *a, **kw: (0, size(out) + size(out) // 3),
-        "gemv_shift": lambda out, x, gain, eps, shift, state, plan, w, *a: (0, nb(w)),
-        "gemv_glu": lambda out, x, z, u, w, *a, **kw: (0, nb(w)),
+        "gemv_pair": lambda out, x, x2, w, *a, **kw: (0, nb(w)),
+        "gemv_add": lambda out, x, w, *a: (0, nb(w)),
+        "gemv_glu": lambda out, z, u, w, *a, **kw: (0, nb(w)),
         "latent_decode": lambda out, q, uk, uv, lat, keys, slot, *a, **kw: (0, nb(uk, uv) + int(keys.sum()) * lat.shape[2] * 2),
         "gemv_post": lambda out, x, w, *a, **kw: (0, nb(w)),
         # (every choice streams its expert's matrices; the router's weights are the product in front of it)

@@ -1019,7 +1019,7 @@ def norm_shift(x, gain, eps, pending=None, pending_weight=None, shift=None, stat
         sst = _shift_state(state, plan, D, "norm_shift")
     check(_capi.lib().tv_norm_shift_fwd(
         _p(x), _p(pending), _p(pending_weight), _p(xo), _p(gain), _p(shift), _p(state if shift is not None else None), _p(seq), _p(cu), _p(start), _p(slot),
-        _p(h), _p(hs), T, D, ps, sst, float(eps), _dt(gain), _stream()), "tv_norm_shift_fwd")
+        _p(h), _p(hs), T, D, ps, sst, float(eps), int(plan is not None and plan.decode), _dt(gain), _stream()), "tv_norm_shift_fwd")
     return x if xo is None else xo, h, hs
 
 
@@ -1336,72 +1336,69 @@ def gemv_post(x, weight, prologue=GEMV_NONE, residual=None, norm_weight=None, ep
     return (y, xs, hs) if prologue == GEMV_POSTNORM else y
 
 
-def gemv_shift_takes(rows: int, width: int, dtype) -> bool:
-    """Shapes of tv_gemv_shift_fwd: 1..4 bf16 rows of up to 8 192 elements, twice in LDS."""
-    return dtype == torch.bfloat16 and 1 <= rows <= 4 and width % 8 == 0 and width <= 8192 and rows * width * 4 <= 128 * 1024
+def gemv_rows_take(rows: int, width: int, dtype) -> bool:
+    """Shapes of gemv_pair, gemv_add and gemv_glu: 1..4 bf16 rows that fit the LDS."""
+    return dtype == torch.bfloat16 and 1 <= rows <= 4 and width % 8 == 0 and rows * width * 2 <= 128 * 1024
 
 
-def gemv_shift(x, gain, eps, shift, state, plan, weight, n1, bias=None, pending=None, pending_weight=None):
-    """`norm_shift` and the product behind it for single tokens (1..4): (x', y) with y = [hs @ weight[:n1].T | h @ weight[n1:].T + bias], bf16."""
-    _gpu(x, gain, shift, state, weight, bias, pending, pending_weight)
+def _gemv_rows(what, weight, *rows):
+    if weight.dtype != torch.bfloat16 or weight.dim() != 2 or weight.stride(1) != 1 or any(
+            t.dtype != torch.bfloat16 or t.shape != rows[0].shape or t.shape[1] != weight.shape[1] or t.stride(1) != 1 for t in rows):
+        raise TimeViperHipError(f"{what}: bf16 rows {tuple(rows[0].shape)} against weight {tuple(weight.shape)}")
+
+
+def _bf16_bias(t, n, what):
+    if t is not None:
+        _vec(t, n, what)
+        if t.dtype != torch.bfloat16:
+            raise TimeViperHipError(f"{what}: bf16")
+
+
+def gemv_pair(x, x2, weight, n1, bias=None, act_out=None):
+    """Both input products of a parallel layer for 1..4 bf16 rows, one launch: y = x @ weight[:n1].T (returned) and, when weight has more
+    rows (gate | up), act_out = gelu_tanh(x2 @ gate.T + b) * (x2 @ up.T + b), bias = their biases."""
+    _gpu(x, x2, weight, bias, act_out)
     M, D = x.shape
-    N = weight.shape[0]
-    bf = torch.bfloat16
-    if (x.dtype != torch.float32 or not x.is_contiguous() or weight.dtype != bf or weight.shape[1] != D or weight.stride(1) != 1 or gain.dtype != bf
-            or gain.numel() != 1 or shift.dtype != bf or not plan.decode or (bias is not None and bias.dtype != bf)):
-        raise TimeViperHipError(f"gemv_shift: dense fp32 rows {tuple(x.shape)} against a bf16 weight {tuple(weight.shape)}")
-    _vec(shift, D, "gemv_shift shift")
-    if bias is not None:
-        _vec(bias, N - n1, "gemv_shift bias")
-    xo, ps = None, 0
-    if pending is not None:
-        if pending.shape != x.shape or pending.dtype != bf or pending.stride(1) != 1 or pending_weight.dtype != bf:
-            raise TimeViperHipError("gemv_shift: pending rows and weight in bf16, of x's width")
-        _vec(pending_weight, D, "gemv_shift pending weight")
-        xo, ps = torch.empty_like(x), pending.stride(0)
-    _, _, start, slot = _plan(plan, M, "gemv_shift")
-    sst = _shift_state(state, plan, D, "gemv_shift")
-    y = torch.empty((M, N), dtype=bf, device=x.device)
-    check(_capi.lib().tv_gemv_shift_fwd(
-        _p(x), _p(pending), _p(pending_weight), _p(xo), _p(gain), _p(shift), _p(state), _p(start), _p(slot), _p(weight), _p(bias), _p(y), M, N, int(n1),
-        D, ps, sst, weight.stride(0), N, float(eps), _stream()), "tv_gemv_shift_fwd")
-    return x if xo is None else xo, y
+    ff = (weight.shape[0] - n1) // 2
+    _gemv_rows("gemv_pair", weight, x, *((x2,) if ff else ()))
+    if weight.shape[0] != n1 + 2 * ff or n1 < 1 or (ff and (bias is None or act_out is None or act_out.shape != (M, ff) or act_out.dtype != x.dtype
+                                                          or act_out.stride(1) != 1)):
+        raise TimeViperHipError(f"gemv_pair: weight rows {n1} + 2 x {ff}, biases and an (M, {ff}) output for the second part")
+    if ff:
+        _bf16_bias(bias, 2 * ff, "gemv_pair bias")
+    y = torch.empty((M, n1), dtype=x.dtype, device=x.device)
+    check(_capi.lib().tv_gemv_pair_fwd(_p(x), _p(x2) if ff else None, _p(weight), _p(bias), _p(y), _p(act_out) if ff else None, M, int(n1), ff, D,
+                                       x.stride(0), x2.stride(0) if ff else 0, weight.stride(0), n1, act_out.stride(0) if ff else 0, _stream()),
+          "tv_gemv_pair_fwd")
+    return y
 
 
-def gemv_glu_takes(rows: int, k1: int, k2: int, dtype) -> bool:
-    """Shapes of tv_gemv_glu_fwd."""
-    return dtype == torch.bfloat16 and 1 <= rows <= 4 and k1 % 8 == 0 and k2 % 8 == 0 and rows * (k1 + k2) * 2 <= 128 * 1024
+def gemv_add(x, weight, residual, bias=None):
+    """(residual + x @ weight.T + bias in fp32, its bf16 rounding) for 1..4 bf16 rows; residual (M, N) fp32"""
+    _gpu(x, weight, bias, residual)
+    _gemv_rows("gemv_add", weight, x)
+    M, N = x.shape[0], weight.shape[0]
+    _bf16_bias(bias, N, "gemv_add bias")
+    if residual.dtype != torch.float32 or residual.shape != (M, N) or not residual.is_contiguous():
+        raise TimeViperHipError("gemv_add: a dense fp32 residual (M, N)")
+    xo, h = torch.empty_like(residual), torch.empty((M, N), dtype=x.dtype, device=x.device)
+    check(_capi.lib().tv_gemv_add_fwd(_p(x), _p(weight), _p(bias), _p(residual), _p(xo), _p(h), M, N, x.shape[1], x.stride(0), weight.stride(0),
+                                      _stream()), "tv_gemv_add_fwd")
+    return xo, h
 
 
-def gemv_glu(x, z, u, weight, bias=None, residual=None, ids=None):
-    """y = [x | gelu_tanh(z) * u] @ weight.T + bias for 1..4 bf16 rows; x or (z, u) may be None; `ids` (int64): row m meets u[ids[m]].  With
-    `residual` (fp32): (residual + y in fp32, its bf16 rounding), else y in bf16."""
-    _gpu(x, z, u, weight, bias, residual, ids)
-    bf = torch.bfloat16
-    M = (x if x is not None else z).shape[0]
-    N, Kd = weight.shape
-    k1 = 0 if x is None else x.shape[1]
-    if (k1 + (0 if z is None else z.shape[1]) != Kd or weight.dtype != bf or weight.stride(1) != 1 or (z is None) != (u is None)
-            or any(t is not None and (t.dtype != bf or t.stride(1) != 1) for t in (x, z, u)) or any(t is not None and t.shape[0] != M for t in (x, z))
-            or (u is not None and (u.shape[1] != z.shape[1] or (ids is None and u.shape[0] != M)))
+def gemv_glu(z, u, weight, ids=None):
+    """(gelu_tanh(z) * u) @ weight.T for 1..4 bf16 rows; `ids` (int64): row m meets u[ids[m]]"""
+    _gpu(z, u, weight, ids)
+    _gemv_rows("gemv_glu", weight, z)
+    M, N = z.shape[0], weight.shape[0]
+    if (u.dtype != z.dtype or u.stride(1) != 1 or u.shape[1] != z.shape[1] or (ids is None and u.shape[0] != M)
             or (ids is not None and (ids.dtype != torch.int64 or ids.numel() != M or not ids.is_contiguous()))):
-        raise TimeViperHipError(f"gemv_glu: bf16 rows that make up the {Kd} columns of the weight")
-    if bias is not None:
-        _vec(bias, N, "gemv_glu bias")
-        if bias.dtype != bf:
-            raise TimeViperHipError("gemv_glu: bf16 bias")
-    y = xo = ho = None
-    if residual is not None:
-        if residual.dtype != torch.float32 or residual.shape != (M, N) or not residual.is_contiguous():
-            raise TimeViperHipError("gemv_glu: a dense fp32 residual (M, N)")
-        xo, ho = torch.empty_like(residual), torch.empty((M, N), dtype=bf, device=residual.device)
-    else:
-        y = torch.empty((M, N), dtype=bf, device=weight.device)
-    st = lambda t: 0 if t is None else t.stride(0)
-    check(_capi.lib().tv_gemv_glu_fwd(
-        _p(x), _p(z), _p(u), _p(ids), 0 if u is None else u.shape[0], _p(weight), _p(bias), _p(residual), _p(xo), _p(ho), _p(y), M, N, k1, Kd, st(x),
-        st(z), st(u), weight.stride(0), N, _stream()), "tv_gemv_glu_fwd")
-    return y if residual is None else (xo, ho)
+        raise TimeViperHipError("gemv_glu: u rows of z's width, one per row or by int64 ids")
+    y = torch.empty((M, N), dtype=z.dtype, device=z.device)
+    check(_capi.lib().tv_gemv_glu_fwd(_p(z), _p(u), _p(ids), u.shape[0], _p(weight), _p(y), M, N, z.shape[1], z.stride(0), u.stride(0), weight.stride(0),
+                                      N, _stream()), "tv_gemv_glu_fwd")
+    return y
 
 
 # ------------------------------------------------- mixture of experts

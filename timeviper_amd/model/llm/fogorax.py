@@ -100,8 +100,7 @@ class FogoraxModel(nn.Module):
         self.final_gain = _weight()
 
     def _fused(self, ids, plan) -> bool:
-        """Single tokens of up to four sequences run on the matrix-vector kernels, with norms, shift, activations and residual adds
-        inside them; TV_DECODE_FUSED=0 keeps the general operators."""
+        """Single tokens of up to four sequences run on the matrix-vector kernels, with activations and residual adds inside them; TV_DECODE_FUSED=0 keeps the general operators."""
         return (plan.decode and os.environ.get("TV_DECODE_FUSED", "1") != "0"
                 and all(l.decode_takes(ids.numel(), self.final_gain.dtype) for l in self.layers))
 

@@ -52,7 +52,7 @@ class TokenSide(nn.Module):
         return F.linear(K.gated_mul(F.linear(h, self.gate), rows, K.ACT_GELU_TANH, ids=ids), self.proj)
 
     def decode(self, h, ids, rows):
-        return K.gemv_glu(None, K.gemv_post(h, self.gate), rows, self.proj, ids=ids)
+        return K.gemv_glu(K.gemv_post(h, self.gate), rows, self.proj, ids=ids)
 
 
 class ParallelLayer(nn.Module):
@@ -87,15 +87,15 @@ class ParallelLayer(nn.Module):
         return x, (self.side(h, ids, side_rows), self.side.norm)
 
     def decode_takes(self, rows, dtype):
-        D, k2 = self.shift.numel(), self.out.shape[1] - self.k1
-        return (K.gemv_shift_takes(rows, D, dtype) and K.gemv_post_takes(rows, D, dtype) and K.gemv_glu_takes(rows, self.k1, k2, dtype)
-                and K.gemv_glu_takes(rows, 0, self.side.dim, dtype))
+        return all(K.gemv_rows_take(rows, n, dtype) for n in (self.shift.numel(), self.out.shape[1], self.side.dim)) and self.k1 % 8 == 0
 
     def decode(self, x, pending, ids, side_rows, state, kv_rows, plan):
-        """The same for a few single tokens: norms, shift, activations and residual adds inside the matrix-vector products."""
+        """The same for a few single tokens on matrix-vector kernels: both input products and the activation in one launch, the residual
+        add behind the output product."""
         y, w = pending or (None, None)
-        x, p = K.gemv_shift(x, self.gain, self.eps, self.shift, state, plan, self.inp, self.n1, self.inp_bias, y, w)
-        o = self.mixer.attend(p[:, :self.n1], kv_rows, plan)
-        gate, up = self.mlp.split(p[:, self.n1:]) if self.mlp is not None else (None, None)
-        x, h = K.gemv_glu(o, gate, up, self.out, self.out_bias, residual=x)
+        x, h, hs = K.norm_shift(x, self.gain, self.eps, y, w, self.shift, state, plan, need_h=self.mlp is not None)
+        u = torch.empty((x.shape[0], self.out.shape[1]), dtype=hs.dtype, device=hs.device)
+        p = K.gemv_pair(hs, h, self.inp, self.n1, self.inp_bias, act_out=u[:, self.k1:])
+        self.mixer.attend(p, kv_rows, plan, out=u[:, :self.k1])
+        x, h = K.gemv_add(u, self.out, x, self.out_bias)
         return x, (self.side.decode(h, ids, side_rows), self.side.norm)
