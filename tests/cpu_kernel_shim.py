@@ -269,7 +269,7 @@ def _moe_combine(expert_out, pos, weights, residual, norm_weight, eps, weight_of
     return _rms_ex(u, norm_weight, eps, weight_offset, residual=residual, mult=mult, out_dtype=out_dtype)
 
 
-def _embed(ids, table, scale=1.0, positions=None, plan=None):
+def _embed(ids, table, scale=1.0, positions=None, plan=None, need_h=True):
     x = table[ids.reshape(-1)].float() * scale
     if positions is not None:
         x = x + positions[_places(plan)].float()

@@ -28,6 +28,8 @@ CONFIGS = {
                                layer(8, 4, 128, 128, 300, 0, 384, kv_from=0)], 64),
     # one of everything; a window of one token, nothing kept
     "ones": config(97, 64, [layer(1, 1, 32, 32, 1, 0, 32, scale=1.0), layer(1, 1, 8, 8, 2, 1, None, scale=1.0)], 8, positions=40, eps=1e-6),
+    # rows the matrix-vector kernels take around heads the attention kernels do not
+    "mixed": config(75, 64, [layer(2, 2, 20, 12, 11, 2, 40), layer(4, 2, 12, 18, 30, 0, 24), layer(2, 2, 20, 12, 300, 0, 16, kv_from=0)], 16),
     # heads wider than the prompt kernel's tiles; everything visible
     "wide": config(80, 128, [layer(2, 1, 192, 256, 500, 0, 72), layer(3, 3, 256, 136, 17, 4, None)], 16),
 }

@@ -356,7 +356,8 @@ def test_stream_behind_every_layer(name, tmp_path):
         close(got, w, 2e-5)
 
 
-@pytest.mark.parametrize("name,dtype", [("odd", torch.float32), ("tiles", torch.float32), ("large", torch.float32), ("tiles", BF), ("large", BF)])
+@pytest.mark.parametrize("name,dtype", [("odd", torch.float32), ("tiles", torch.float32), ("large", torch.float32), ("tiles", BF), ("large", BF),
+                                        ("mixed", BF)])
 @pytest.mark.parametrize("cuts", [[2] * 30, [1] * 70, [64, 1, 1, 3], [7, 2, 2, 1, 33, 5], [127, 2]])
 def test_portions_of_a_prompt(name, dtype, cuts, tmp_path):
     from timeviper_amd.model.llm import TextEngine

@@ -147,7 +147,7 @@ def op_table(K):
         "residual_add": lambda out, x, u: (0, nb(x, u) + size(out)),
         "gated_mul": lambda res, a, b, *r, **kw: (0, 3 * nb(a)),
         "scatter_rows": lambda out, src, *a: (0, 2 * nb(src)),
-        "embed_scaled": lambda out, ids, *a, **kw: (0, size(out) + size(out) // 3),
+        "embed_scaled": lambda out, ids, table, *a, **kw: (0, size(out) + 2 * ids.numel() * table.shape[1] * 2),      # a table row and a position row
         "gemv_pair": lambda out, x, x2, w, *a, **kw: (0, nb(w)),
         "gemv_add": lambda out, x, w, *a: (0, nb(w)),
         "gemv_glu": lambda out, z, u, w, *a, **kw: (0, nb(w)),

@@ -953,7 +953,7 @@ def moe_combine_norm(expert_out, pos, weights, residual, norm_weight, eps, weigh
     return y, s
 
 
-def embed_scaled(ids, table, scale=1.0, positions=None, plan=None):
+def embed_scaled(ids, table, scale=1.0, positions=None, plan=None, need_h=True):
     """(fp32 rows, rows in the table's dtype) of `table[ids] * scale`; ids int64 on the GPU.  `positions` (max, D): the row of the
     token's place in its sequence is added (plan: the step's `cache.StepPlan`; its places lie within the table)."""
     _gpu(ids, table, positions)
@@ -962,7 +962,7 @@ def embed_scaled(ids, table, scale=1.0, positions=None, plan=None):
     if flat.dtype != torch.int64 or not table.is_contiguous():
         raise TimeViperHipError("embed_scaled: int64 ids and a contiguous table")
     x = torch.empty((flat.numel(), D), dtype=torch.float32, device=table.device)
-    h = torch.empty((flat.numel(), D), dtype=table.dtype, device=table.device)
+    h = torch.empty((flat.numel(), D), dtype=table.dtype, device=table.device) if need_h else None
     seq = cu = start = None
     if positions is not None:
         seq, cu, start = _plan(plan, flat.numel(), "embed_scaled")[:3]

@@ -11,9 +11,9 @@ memory (`HybridMambaAttentionDynamicCache.begin_static_decode`), the attention k
 tokens, and replayed per token with one `hipGraphLaunch`.
 
 Valid for stacks whose decode step does not depend on the host-side position (`llm.graph_decode_supported(cache)`): the
-Nemotron-H hybrid has no positional encoding (modeling_nano.py:1012-1220), nor has Fasovik, whose slots, positions and key
-counts are device tensors anyway; a rotary backbone (Qwen2) would bake its angle in — `GraphedDecodeStep` is not
-offered for it.  The cache side is the `StaticDecode` contract of cache.py.
+Nemotron-H hybrid has no positional encoding (modeling_nano.py:1012-1220), nor has Fasovik, and the packed models (packed.py;
+Fogorax has learned positions) keep slots, positions and key counts in device tensors; a rotary backbone (Qwen2) would bake its
+angle in — `GraphedDecodeStep` is not offered for it.  The cache side is the `StaticDecode` contract of cache.py.
 """
 from __future__ import annotations
 

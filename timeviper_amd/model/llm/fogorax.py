@@ -106,7 +106,7 @@ class FogoraxModel(nn.Module):
 
     def forward(self, ids, cache: SlotStateCache, plan, trace: Optional[list] = None):
         """x (T, width) fp32 and what still waits for it"""
-        x = K.embed_scaled(ids, self.embed.weight, positions=self.positions, plan=plan)[0]
+        x = K.embed_scaled(ids, self.embed.weight, positions=self.positions, plan=plan, need_h=False)[0]
         pending, side = None, self.side_embed.split(self.config.side_dim, dim=1)
         fused = trace is None and self._fused(ids, plan)
         if trace is not None:
