@@ -166,7 +166,7 @@ __global__ __launch_bounds__(RX_THREADS) void embed_scaled_kernel(const int64_t*
                                                                   float* __restrict__ x, T* __restrict__ h, int D, int64_t vocab,
                                                                   float scale, const T* __restrict__ pos, const int* __restrict__ seq,
                                                                   const int* __restrict__ cu, const int* __restrict__ start,
-                                                                  int64_t max_pos) {
+                                                                  int64_t max_pos, int vec) {
   const int64_t row = blockIdx.x, id = ids[row];
   const bool ok = id >= 0 && id < vocab;             // (callers check on the host; a bad id or place reads nothing)
   int64_t at = -1;
@@ -174,6 +174,22 @@ __global__ __launch_bounds__(RX_THREADS) void embed_scaled_kernel(const int64_t*
     const int b = seq[row];
     at = (int64_t)start[b] + row - cu[b];
     if (at >= max_pos) at = -1;
+  }
+  if (vec) {
+    for (int iv = threadIdx.x; iv < D / 8; iv += RX_THREADS) {
+      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, p[8];
+      if (ok) load8<T>(table + id * D + 8 * iv, v);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] *= scale;
+      if (at >= 0) {
+        load8<T>(pos + at * D + 8 * iv, p);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] += p[i];
+      }
+      store8<float>(x + row * D + 8 * iv, v);
+      if (h) store8<T>(h + row * D + 8 * iv, v);
+    }
+    return;
   }
   for (int d = threadIdx.x; d < D; d += RX_THREADS) {
     float v = ok ? to_f32(table[id * D + d]) * scale : 0.f;
@@ -241,10 +257,11 @@ extern "C" int tv_embed_scaled_fwd(const int64_t* ids, const void* table, float*
   TV_CHECK_ARG(ids && table && x && (!pos || (seq && cu && start && max_pos > 0)), "embed_scaled: null pointer");
   hipStream_t st = (hipStream_t)stream;
   const dim3 grid((unsigned)rows);
+  const int vec = D % 8 == 0 && al16(table) && al16(x) && al16(h) && al16(pos);
   if (dtype == TV_F32)
-    embed_scaled_kernel<float><<<grid, RX_THREADS, 0, st>>>(ids, (const float*)table, x, (float*)h, D, vocab, scale, (const float*)pos, seq, cu, start, max_pos);
+    embed_scaled_kernel<float><<<grid, RX_THREADS, 0, st>>>(ids, (const float*)table, x, (float*)h, D, vocab, scale, (const float*)pos, seq, cu, start, max_pos, vec);
   else if (dtype == TV_BF16)
-    embed_scaled_kernel<bf16_t><<<grid, RX_THREADS, 0, st>>>(ids, (const bf16_t*)table, x, (bf16_t*)h, D, vocab, scale, (const bf16_t*)pos, seq, cu, start, max_pos);
+    embed_scaled_kernel<bf16_t><<<grid, RX_THREADS, 0, st>>>(ids, (const bf16_t*)table, x, (bf16_t*)h, D, vocab, scale, (const bf16_t*)pos, seq, cu, start, max_pos, vec);
   else TV_UNSUPPORTED("embed_scaled: dtype %d", dtype);
   TV_LAUNCH_CHECK();
 }
